@@ -6,6 +6,7 @@ from .gokazen import GokazenConfig
 from .pudorax import PudoraxConfig
 from .dupidra import DupidraConfig
 from .vepelix import VepelixConfig
+from .lurepel import LurepelConfig
 
 __all__ = ["ConfigError", "ConfigReader", "architecture_name", "read_config_json", "LayerKinds", "Qwen3Config", "GokazenConfig", "PudoraxConfig",
-           "DupidraConfig", "VepelixConfig"]
+           "DupidraConfig", "VepelixConfig", "LurepelConfig"]

@@ -23,6 +23,20 @@ __device__ inline bf16_t from_f32<bf16_t>(float x) {
   return r;
 }
 
+// ---- gated activations ----------------------------------------------------------------------
+// act(gate) * up with act(g) = g / (1 + exp(-g (slope + cube g^2))): silu with slope 1 and cube 0, and with slope
+// 2 sqrt(2/pi) and cube 2 sqrt(2/pi) 0.044715 the tanh form of GELU, since (1 + tanh(y)) / 2 = 1 / (1 + exp(-2y)).
+struct GateForm {
+  float slope, cube;
+};
+enum BhGate { BH_GATE_SILU = 1, BH_GATE_GELU_TANH = 2 };
+inline GateForm bh_gate_form(int gate) {
+  return gate == BH_GATE_GELU_TANH ? GateForm{1.5957691216057308f, 1.5957691216057308f * 0.044715f} : GateForm{1.0f, 0.0f};
+}
+__device__ inline float gate_mul(float gate, float up, GateForm form) {
+  return gate / (1.0f + expf(-gate * fmaf(form.cube, gate * gate, form.slope))) * up;
+}
+
 // ---- reductions -------------------------------------------------------------------------
 
 __device__ inline float wave_sum(float v) {

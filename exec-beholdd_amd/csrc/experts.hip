@@ -8,6 +8,10 @@
 //               (an infinite limit, alpha 1 and shift 0 give silu(g) * u)
 // A router may score by the sigmoid of every chosen logit instead (`scoring` 1), and a pair's weight may multiply the
 // expert's input instead of its output: W (w h) = w (W h), so the gate and up sums are multiplied ahead of the activation.
+// A router may also score by each expert's share of the softmax over all of them (`scoring` 2), choose by these scores plus a
+// learned correction and weigh by the scores alone, and may count experts without matrices behind the E with: what such an
+// expert gives is the input h itself, so the kernels with matrices leave its pairs out and those that add a row's shares up
+// (experts_down, experts_combine) add weight * h in its place.
 // Router logits, the softmax and all sums are float32.
 #include "common.h"
 
@@ -23,8 +27,8 @@ __device__ inline float clamped_glu(float g, float u, float limit, float alpha, 
 // One wave a row: a lane holds the logits of experts lane, lane + 64, ...; the largest is found `top` times over, each time
 // without those already taken (ties go to the lower index).
 __global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restrict__ logits, const float* __restrict__ bias,
-                                                         int32_t* __restrict__ chosen, float* __restrict__ weights, int n_rows,
-                                                         int E, int top, int scoring) {
+                                                         const float* __restrict__ correction, int32_t* __restrict__ chosen,
+                                                         float* __restrict__ weights, int n_rows, int E, int top, int scoring) {
   const int lane = threadIdx.x & (BH_WAVE - 1), row = blockIdx.x * (blockDim.x / BH_WAVE) + threadIdx.x / BH_WAVE;
   if (row >= n_rows) return;
   const float* z = logits + (size_t)row * E;
@@ -33,6 +37,25 @@ __global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restric
   for (int i = 0; i < ROUTE_PER_LANE; ++i) {
     const int e = lane + i * BH_WAVE;
     v[i] = e < E ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
+  }
+  float score[ROUTE_PER_LANE];      // scoring 2: the share without the correction; v becomes the number to choose by
+  if (scoring == 2) {
+    float top_z = -INFINITY, total = 0.f;
+#pragma unroll
+    for (int i = 0; i < ROUTE_PER_LANE; ++i) top_z = fmaxf(top_z, v[i]);
+    top_z = wave_max(top_z);
+#pragma unroll
+    for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+      score[i] = lane + i * BH_WAVE < E ? expf(v[i] - top_z) : 0.f;
+      total += score[i];
+    }
+    total = wave_sum(total);
+#pragma unroll
+    for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+      const int e = lane + i * BH_WAVE;
+      score[i] /= total;
+      if (e < E) v[i] = score[i] + (correction ? correction[e] : 0.f);
+    }
   }
   unsigned taken = 0;      // bit i: this lane's expert lane + 64 i was chosen
   float largest = 0.f, sum = 0.f, mine = 0.f;      // lane j keeps the j-th choice's exponential
@@ -59,7 +82,16 @@ __global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restric
     }
     if ((best_e & (BH_WAVE - 1)) == lane) taken |= 1u << (best_e / BH_WAVE);
     if (j == 0) largest = best;
-    const float p = scoring ? 1.0f / (1.0f + expf(-best)) : expf(best - largest);
+    float p;
+    if (scoring == 2) {
+      float own = 0.f;
+#pragma unroll
+      for (int i = 0; i < ROUTE_PER_LANE; ++i)
+        if (i == best_e / BH_WAVE) own = score[i];
+      p = __shfl(own, best_e & (BH_WAVE - 1), BH_WAVE);
+    } else {
+      p = scoring ? 1.0f / (1.0f + expf(-best)) : expf(best - largest);
+    }
     sum += p;
     if (lane == j) {
       mine = p;
@@ -72,11 +104,12 @@ __global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restric
   }
 }
 
-extern "C" int bh_route_top_k(const float* logits, const float* bias, int32_t* chosen, float* weights, int n_rows, int E, int top,
+extern "C" int bh_route_top_k(const float* logits, const float* bias, const float* correction, int32_t* chosen, float* weights, int n_rows, int E, int top,
                               int scoring, hipStream_t stream) {
   BH_REQUIRE(n_rows > 0 && E > 0 && E <= BH_WAVE * ROUTE_PER_LANE, "route_top_k: 1 to %d experts, got %d", BH_WAVE * ROUTE_PER_LANE, E);
   BH_REQUIRE(top >= 1 && top <= E && top <= ROUTE_MAX_TOP, "route_top_k: 1 to min(%d, %d) experts a row, got %d", E, ROUTE_MAX_TOP, top);
-  route_top_k_kernel<<<(n_rows + 3) / 4, 256, 0, stream>>>(logits, bias, chosen, weights, n_rows, E, top, scoring);
+  BH_REQUIRE(scoring >= 0 && scoring <= 2 && (correction == nullptr || scoring == 2), "route_top_k: scoring %d, or a correction that does not go with it", scoring);
+  route_top_k_kernel<<<(n_rows + 3) / 4, 256, 0, stream>>>(logits, bias, correction, chosen, weights, n_rows, E, top, scoring);
   return bh_check_launch("route_top_k");
 }
 
@@ -103,11 +136,12 @@ __device__ inline float wave_dot(const T* __restrict__ w, const float* __restric
 // grid (pairs, ceil(ff / EX_OUTS)); w_gu [E][2 ff][K]: an expert's gate rows, then its up rows.
 template <typename T>
 __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restrict__ h, const int32_t* __restrict__ chosen,
-                                                              const T* __restrict__ w_gu, T* __restrict__ inner, int top, int K, int ff,
+                                                              const T* __restrict__ w_gu, T* __restrict__ inner, int top, int E, int K, int ff,
                                                               float limit, float alpha, float shift,
                                                               const float* __restrict__ in_weights) {
   extern __shared__ float xs[];
   const int pair = blockIdx.x, row = pair / top, e = chosen[pair];
+  if (e >= E) return;      // an expert without matrices
   for (int k = threadIdx.x; k < K; k += blockDim.x) xs[k] = to_f32(h[(size_t)row * K + k]);
   __syncthreads();
   const int lane = threadIdx.x & (BH_WAVE - 1), wave = threadIdx.x / BH_WAVE;
@@ -123,7 +157,7 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
 }
 
 extern "C" int bh_experts_gate_up(const void* h, int dtype, const int32_t* chosen, const void* w_gu, void* inner, int n_rows, int top,
-                                  int K, int ff, float limit, float alpha, float shift, const float* in_weights, hipStream_t stream) {
+                                  int E, int K, int ff, float limit, float alpha, float shift, const float* in_weights, hipStream_t stream) {
   BH_REQUIRE(n_rows > 0 && top > 0 && K > 0 && ff > 0, "experts_gate_up: sizes must be positive");
   BH_REQUIRE((size_t)K * sizeof(float) <= 64 * 1024, "experts_gate_up: rows of up to 16384 inputs, got %d", K);
   dim3 grid(n_rows * top, (ff + EX_OUTS - 1) / EX_OUTS);
@@ -131,10 +165,10 @@ extern "C" int bh_experts_gate_up(const void* h, int dtype, const int32_t* chose
   if (dtype == BH_F32) bh_allow_lds<experts_gate_up_kernel<float>>(lds);
   if (dtype == BH_BF16) bh_allow_lds<experts_gate_up_kernel<bf16_t>>(lds);
   if (dtype == BH_F32)
-    experts_gate_up_kernel<float><<<grid, 64 * EX_WAVES, lds, stream>>>((const float*)h, chosen, (const float*)w_gu, (float*)inner, top, K, ff,
+    experts_gate_up_kernel<float><<<grid, 64 * EX_WAVES, lds, stream>>>((const float*)h, chosen, (const float*)w_gu, (float*)inner, top, E, K, ff,
                                                                        limit, alpha, shift, in_weights);
   else if (dtype == BH_BF16)
-    experts_gate_up_kernel<bf16_t><<<grid, 64 * EX_WAVES, lds, stream>>>((const bf16_t*)h, chosen, (const bf16_t*)w_gu, (bf16_t*)inner, top, K,
+    experts_gate_up_kernel<bf16_t><<<grid, 64 * EX_WAVES, lds, stream>>>((const bf16_t*)h, chosen, (const bf16_t*)w_gu, (bf16_t*)inner, top, E, K,
                                                                         ff, limit, alpha, shift, in_weights);
   else
     return bh_fail("experts_gate_up: unknown dtype %d", dtype);
@@ -145,7 +179,8 @@ extern "C" int bh_experts_gate_up(const void* h, int dtype, const int32_t* chose
 template <typename T>
 __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__ inner, const int32_t* __restrict__ chosen,
                                                            const float* __restrict__ weights, const T* __restrict__ w_d,
-                                                           float* __restrict__ hidden, int top, int ff, int D) {
+                                                           float* __restrict__ hidden, const T* __restrict__ through, int top, int E,
+                                                           int ff, int D, int fresh) {
   extern __shared__ float xs[];      // [top][ff]
   const int row = blockIdx.x;
   for (int k = threadIdx.x; k < top * ff; k += blockDim.x) xs[k] = to_f32(inner[(size_t)row * top * ff + k]);
@@ -157,14 +192,15 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
     float total = 0.f;
     for (int j = 0; j < top; ++j) {
       const int e = chosen[(size_t)row * top + j];
-      total = fmaf(weights ? weights[(size_t)row * top + j] : 1.0f, wave_dot(w_d + ((size_t)e * D + o) * ff, xs + (size_t)j * ff, ff, lane), total);
+      const float share = e >= E ? to_f32(through[(size_t)row * D + o]) : wave_dot(w_d + ((size_t)e * D + o) * ff, xs + (size_t)j * ff, ff, lane);
+      total = fmaf(weights ? weights[(size_t)row * top + j] : 1.0f, share, total);
     }
-    if (lane == 0) hidden[(size_t)row * D + o] += total;
+    if (lane == 0) hidden[(size_t)row * D + o] = fresh ? total : hidden[(size_t)row * D + o] + total;
   }
 }
 
 extern "C" int bh_experts_down(const void* inner, int dtype, const int32_t* chosen, const float* weights, const void* w_d, float* hidden,
-                               int n_rows, int top, int ff, int D, hipStream_t stream) {
+                               const void* through, int n_rows, int top, int E, int ff, int D, int fresh, hipStream_t stream) {
   BH_REQUIRE(n_rows > 0 && top > 0 && ff > 0 && D > 0, "experts_down: sizes must be positive");
   const size_t lds = (size_t)top * ff * sizeof(float);
   BH_REQUIRE(lds <= 64 * 1024, "experts_down: %d experts a row of %d inner values do not fit the local memory", top, ff);
@@ -172,10 +208,11 @@ extern "C" int bh_experts_down(const void* inner, int dtype, const int32_t* chos
   if (dtype == BH_F32) bh_allow_lds<experts_down_kernel<float>>(lds);
   if (dtype == BH_BF16) bh_allow_lds<experts_down_kernel<bf16_t>>(lds);
   if (dtype == BH_F32)
-    experts_down_kernel<float><<<grid, 64 * EX_WAVES, lds, stream>>>((const float*)inner, chosen, weights, (const float*)w_d, hidden, top, ff, D);
+    experts_down_kernel<float><<<grid, 64 * EX_WAVES, lds, stream>>>((const float*)inner, chosen, weights, (const float*)w_d, hidden, (const float*)through, top,
+                                                                   E, ff, D, fresh);
   else if (dtype == BH_BF16)
-    experts_down_kernel<bf16_t><<<grid, 64 * EX_WAVES, lds, stream>>>((const bf16_t*)inner, chosen, weights, (const bf16_t*)w_d, hidden, top, ff,
-                                                                     D);
+    experts_down_kernel<bf16_t><<<grid, 64 * EX_WAVES, lds, stream>>>((const bf16_t*)inner, chosen, weights, (const bf16_t*)w_d, hidden, (const bf16_t*)through,
+                                                                    top, E, ff, D, fresh);
   else
     return bh_fail("experts_down: unknown dtype %d", dtype);
   return bh_check_launch("experts_down");
@@ -395,23 +432,37 @@ extern "C" int bh_experts_gather(const void* x, int dtype, int top, const int32_
   return bh_check_launch("experts_gather");
 }
 
-// y [*][D] float32: the result of pair p lies at row place[p] (or p where no places are given).
+// y [*][D] float32: the result of pair p lies at row place[p] (or p where no places are given).  With `through` (the rows'
+// inputs [rows][D], in the activations' type) a pair whose expert is numbered E or higher gives its row's input instead.
+// `fresh`: the sum is written, not added.
+template <typename T>
 __global__ __launch_bounds__(256) void experts_combine_kernel(const float* __restrict__ y, const int32_t* __restrict__ place,
-                                                              const float* __restrict__ weights, float* __restrict__ hidden, int top, int D) {
+                                                              const float* __restrict__ weights, float* __restrict__ hidden,
+                                                              const T* __restrict__ through, const int32_t* __restrict__ chosen, int E,
+                                                              int top, int D, int fresh) {
   const int row = blockIdx.x, d = blockIdx.y * blockDim.x + threadIdx.x;
   if (d >= D) return;
   float total = 0.f;
   for (int j = 0; j < top; ++j) {
     const int pair = row * top + j;
-    total = fmaf(weights ? weights[pair] : 1.0f, y[(size_t)(place ? place[pair] : pair) * D + d], total);
+    const bool passes = through && chosen[pair] >= E;
+    const float share = passes ? to_f32(through[(size_t)row * D + d]) : y[(size_t)(place ? place[pair] : pair) * D + d];
+    total = fmaf(weights ? weights[pair] : 1.0f, share, total);
   }
-  hidden[(size_t)row * D + d] += total;
+  hidden[(size_t)row * D + d] = fresh ? total : hidden[(size_t)row * D + d] + total;
 }
 
-extern "C" int bh_experts_combine(const float* y, const int32_t* place, const float* weights, float* hidden, int n_rows, int top, int D,
-                                  hipStream_t stream) {
+extern "C" int bh_experts_combine(const float* y, const int32_t* place, const float* weights, float* hidden, const void* through,
+                                  int dtype, const int32_t* chosen, int E, int n_rows, int top, int D, int fresh, hipStream_t stream) {
   BH_REQUIRE(n_rows > 0 && top > 0 && D > 0, "experts_combine: sizes must be positive");
   BH_REQUIRE((D + 255) / 256 <= 65535, "experts_combine: rows of up to 16 million outputs");
-  experts_combine_kernel<<<dim3(n_rows, (D + 255) / 256), 256, 0, stream>>>(y, place, weights, hidden, top, D);
+  BH_REQUIRE(through == nullptr || (chosen != nullptr && E > 0), "experts_combine: inputs that are handed through come with the choices");
+  const dim3 grid(n_rows, (D + 255) / 256);
+  if (dtype == BH_F32)
+    experts_combine_kernel<float><<<grid, 256, 0, stream>>>(y, place, weights, hidden, (const float*)through, chosen, E, top, D, fresh);
+  else if (dtype == BH_BF16)
+    experts_combine_kernel<bf16_t><<<grid, 256, 0, stream>>>(y, place, weights, hidden, (const bf16_t*)through, chosen, E, top, D, fresh);
+  else
+    return bh_fail("experts_combine: unknown dtype %d", dtype);
   return bh_check_launch("experts_combine");
 }

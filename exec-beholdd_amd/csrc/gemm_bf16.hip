@@ -59,8 +59,6 @@ __device__ inline void store_out<bf16_t>(bf16_t* c, size_t at, float v, bool acc
   c[at] = from_f32<bf16_t>(v);
 }
 
-__device__ inline float silu_mul(float gate, float up) { return gate / (1.0f + expf(-gate)) * up; }
-
 // every lane's value of the lane eight further on in its group of 16 (lanes 8 to 15: nothing that matters)
 __device__ inline u32x4_t from_lane_plus_8(u32x4_t v) {
   u32x4_t out;
@@ -117,7 +115,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const uint16_t*
                                                                  const uint16_t* __restrict__ w,
                                                                  TC* __restrict__ c, int M, int N, int K,
                                                                  int accumulate, int pair_blocks,
-                                                                 RidingNorm norm, RowBlocks blocks) {
+                                                                 RidingNorm norm, RowBlocks blocks, GateForm form) {
   __shared__ float partial[WAVES][RT][MB][256];
   __shared__ float row_factor[MB * 16];
   // The norm ahead: 32 threads per row, each with every 32nd partial sum.  The first 256 of a row are asked
@@ -293,7 +291,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const uint16_t*
     float value = 0.f;   // what the residual holds afterwards (norm.behind_weight: float32 output, RT == 1)
     if (valid) {
       if (RT == 2) {
-        store_out<TC>(c, (size_t)bh_rows_index(blocks.c, m, n, N), silu_mul(sum[0], sum[RT - 1]), false);
+        store_out<TC>(c, (size_t)bh_rows_index(blocks.c, m, n, N), gate_mul(sum[0], sum[RT - 1], form), false);
       } else if (OUT_EARLY) {
         value = accumulate ? before[pass] + sum[0] : sum[0];
         reinterpret_cast<float*>(c)[(size_t)m * N + n] = value;
@@ -532,7 +530,7 @@ typedef uint16_t u16x4_t __attribute__((ext_vector_type(4)));
 template <bool SWIGLU, typename TC>
 __global__ __launch_bounds__(256) void gemm_parts_finish_kernel(const float* __restrict__ sums, TC* __restrict__ c,
                                                                 int M, int N, int K, int parts, int accumulate,
-                                                                RidingNorm norm, RowBlocks blocks) {
+                                                                RidingNorm norm, RowBlocks blocks, GateForm form) {
   const int w_rows = SWIGLU ? 2 * N : N;
   const int col = threadIdx.x % 16, n = blockIdx.x * FINISH_COLUMNS + 4 * col, m = blockIdx.y * 16 + threadIdx.x / 16;
   const bool valid = m < M && n < N;
@@ -575,7 +573,7 @@ __global__ __launch_bounds__(256) void gemm_parts_finish_kernel(const float* __r
   if (valid) {
     if (SWIGLU) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) value[i] = silu_mul(first[i], second[i]);
+      for (int i = 0; i < 4; ++i) value[i] = gate_mul(first[i], second[i], form);
     } else {
       value = first;
       if (accumulate) {
@@ -728,7 +726,7 @@ template <bool TILES, bool SWIGLU, int WX, int WY, int WM, int WN, int BUFFERS, 
 __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(const uint16_t* __restrict__ a,
                                                                    const uint16_t* __restrict__ w,
                                                                    TC* __restrict__ c, int M, int N, int K,
-                                                                   int accumulate) {
+                                                                   int accumulate, GateForm form) {
   constexpr int THREADS = 64 * WM * WN;
   constexpr int TBM = 32 * WX * WM, TBN = 32 * WY * WN;
   constexpr int A_PIECES = TBM * 8 / THREADS;   // 16-byte pieces of a slice that one thread stages
@@ -856,7 +854,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(const uint16_t
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           const int m = m0 + wm + x * 32 + 8 * (e / 4) + 4 * (lane / 32) + e % 4;
-          if (m < M) store_out<TC>(c, (size_t)m * N + n, silu_mul(acc[x][y][e], acc[x][y + WY / 2][e]), false);
+          if (m < M) store_out<TC>(c, (size_t)m * N + n, gate_mul(acc[x][y][e], acc[x][y + WY / 2][e], form), false);
         }
       }
     } else {
@@ -888,7 +886,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_whole_kernel(const ui
                                                                          TC* __restrict__ c, int M, int N, int K,
                                                                          int accumulate, RidingNorm norm,
                                                                          float* __restrict__ parts_out,
-                                                                         int slices_per_part) {
+                                                                         int slices_per_part, GateForm form) {
   constexpr int THREADS = 64 * WM * WN;
   constexpr int TBM = 32 * WX * WM, TBN = 32 * WY * WN;
   static_assert(TBM <= THREADS, "one thread per row of the tile adds up the norm's partial sums");
@@ -1106,7 +1104,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_whole_kernel(const ui
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           const int m = m0 + wm + x * 32 + 8 * (e / 4) + 4 * (lane / 32) + e % 4;
-          if (m >= m_own && m < M) store_out<TC>(c, (size_t)m * N + n, silu_mul(acc[x][y][e], acc[x][y + WY / 2][e]), false);
+          if (m >= m_own && m < M) store_out<TC>(c, (size_t)m * N + n, gate_mul(acc[x][y][e], acc[x][y + WY / 2][e], form), false);
         }
       }
     } else {
@@ -1140,7 +1138,7 @@ static int skinny_span_rows(int M, int N, int K) {
 
 template <bool TILES, int RT, typename TC>
 static void launch_skinny(const void* a, const void* w, void* c, int M, int N, int K, int accumulate,
-                          int pair_blocks, const RidingNorm& norm, const RowBlocks& blocks, hipStream_t stream) {
+                          int pair_blocks, const RidingNorm& norm, const RowBlocks& blocks, GateForm form, hipStream_t stream) {
   constexpr int WAVES = 8;
   if constexpr (TILES && RT == 1) {
     if (const int span = skinny_span_rows(M, N, K)) {
@@ -1160,7 +1158,7 @@ static void launch_skinny(const void* a, const void* w, void* c, int M, int N, i
   dim3 grid((N + 15) / 16), block(WAVES * 64);
 #define BH_SKINNY(MB, XB)                                                                                 \
   gemm_skinny_kernel<MB, WAVES, TILES, RT, TC, XB><<<grid, block, 0, stream>>>(                           \
-      (const uint16_t*)a, (const uint16_t*)w, (TC*)c, M, N, K, accumulate, pair_blocks, norm, blocks)
+      (const uint16_t*)a, (const uint16_t*)w, (TC*)c, M, N, K, accumulate, pair_blocks, norm, blocks, form)
   if constexpr (TILES) {   // activations in blocks come with packed weights only, up to SKINNY_UP_TO_ROWS rows
     if (blocks.a == 8) {
       BH_SKINNY(1, 8);
@@ -1265,7 +1263,7 @@ static void tiled_parts(int M, int N, int K, int layout, bool swiglu, int* parts
 
 template <bool TILES, bool SWIGLU, typename TC>
 static void launch_tiled(const void* a, const void* w, void* c, int M, int N, int K, int accumulate,
-                         const RidingNorm& norm, float* parts_out, hipStream_t stream) {
+                         const RidingNorm& norm, float* parts_out, GateForm form, hipStream_t stream) {
   int rows, columns;
   const TiledConfig config = tiled_config(M, N, SWIGLU, &rows, &columns);
   const bool whole = tiled_whole(M, N, K, TILES ? 1 : 0, rows, columns);
@@ -1279,10 +1277,10 @@ static void launch_tiled(const void* a, const void* w, void* c, int M, int N, in
     if (TILES && whole)                                                                                    \
       gemm_tiled_whole_kernel<SWIGLU, WX, WY, WM, WN, BUFFERS, TC><<<grid, block, 0, stream>>>(            \
           (const uint16_t*)a, (const uint16_t*)w, (TC*)c, M, N, K, accumulate, norm, parts_out,            \
-          slices_per_part);                                                                                \
+          slices_per_part, form);                                                                                \
     else                                                                                                   \
       gemm_tiled_kernel<TILES, SWIGLU, WX, WY, WM, WN, BUFFERS, TC><<<grid, block, 0, stream>>>(           \
-          (const uint16_t*)a, (const uint16_t*)w, (TC*)c, M, N, K, accumulate);                            \
+          (const uint16_t*)a, (const uint16_t*)w, (TC*)c, M, N, K, accumulate, form);                      \
   } while (0)
   switch (config) {
     case TILED_256: BH_TILED(2, 4, 4, 2, 2); break;
@@ -1347,7 +1345,8 @@ extern "C" int bh_gemm_bf16_writes_blocked(int M, int N, int K, int layout, int 
   return M <= 64 && !tiled_whole(M, N, K, layout, rows, columns) ? 2 : 0;
 }
 
-// layout: 0 = rows, 1 = tiles.  activation: 0 = none; 1 = SwiGLU (W has 2 * N rows: gate rows then up rows).
+// layout: 0 = rows, 1 = tiles.  activation: 0 = none; 1 = SwiGLU (W has 2 * N rows: gate rows then up rows); to bh_gemm_bf16
+// itself also 2: the same with GELU's tanh form on the gate (BhGate; what the queries say of SwiGLU goes for it too).
 // Bytes of scratch memory that bh_gemm_bf16 wants for this product (0: none).
 // In how many parts of K the tiled kernels (whole tiles, or the kernel whose wave groups take turns) multiply a
 // product when they are given scratch memory (1: in one go).
@@ -1384,7 +1383,9 @@ extern "C" int bh_gemm_bf16(const void* a, const void* w, void* c, int c_dtype, 
   BH_REQUIRE(c_dtype == BH_F32 || c_dtype == BH_BF16, "gemm_bf16: unknown output dtype %d", c_dtype);
   BH_REQUIRE(((uintptr_t)a | (uintptr_t)w) % 16 == 0, "gemm_bf16: operands must be 16-byte aligned");
   BH_REQUIRE(layout == 0 || (layout == 1 && K % 64 == 0), "gemm_bf16: the tiles layout needs K=%d to be a multiple of 64", K);
-  BH_REQUIRE(activation == 0 || activation == 1, "gemm_bf16: unknown activation %d", activation);
+  BH_REQUIRE(activation == 0 || activation == BH_GATE_SILU || activation == BH_GATE_GELU_TANH, "gemm_bf16: unknown activation %d", activation);
+  const GateForm form = bh_gate_form(activation);
+  activation = activation != 0;      // from here on: gated or not
   BH_REQUIRE(activation == 0 || (N % 16 == 0 && !accumulate),
              "gemm_bf16: SwiGLU needs a multiple of 16 outputs (got %d) and no accumulation", N);
   BH_REQUIRE((M + 127) / 128 <= 65535, "gemm_bf16: M=%d needs more than 65535 row tiles", M);
@@ -1420,9 +1421,9 @@ extern "C" int bh_gemm_bf16(const void* a, const void* w, void* c, int c_dtype, 
   const RowBlocks finish_blocks = {0, slices ? c_block_rows : 0, slices ? behind_block_rows : 0};
 #define BH_FINISH(SWIGLU, TC)                                                                                \
   gemm_parts_finish_kernel<SWIGLU, TC><<<finish_grid, 256, 0, stream>>>((const float*)scratch, (TC*)c, M, N, K, \
-                                                                         parts, accumulate, norm, finish_blocks)
+                                                                         parts, accumulate, norm, finish_blocks, form)
   if (!f32 && a_block_rows == 16 && layout == 1 && gemm_slices_gated(M, N, K, activation))   // the SwiGLU of many outputs: no parts, no finishing kernel
-    return gemm_slices_launch_gated(a, w, c, c_block_rows, M, N, K, ahead_ss, ahead_blocks, ahead_eps, stream);
+    return gemm_slices_launch_gated(a, w, c, c_block_rows, M, N, K, ahead_ss, ahead_blocks, ahead_eps, form, stream);
   if (slices) {
     BH_REQUIRE(((uintptr_t)c | (uintptr_t)scratch | (uintptr_t)behind_rows) % 16 == 0,
                "gemm_bf16: output, scratch memory and norm rows must be 16-byte aligned");
@@ -1439,7 +1440,7 @@ extern "C" int bh_gemm_bf16(const void* a, const void* w, void* c, int c_dtype, 
   const int a_blocked = a_block_rows == 16 && !skinny, c_blocked = c_block_rows == 16 && !skinny;
   if (!ahead_ss && !behind_weight && (f32 || !accumulate)) {   // many rows: the kernel whose wave groups take turns
     if (const int blocks = gemm_turns_blocks(M, N, K, layout, activation))
-      return gemm_turns_launch(a, w, c, c_dtype, accumulate, M, N, K, activation, blocks, a_blocked, c_blocked, stream);
+      return gemm_turns_launch(a, w, c, c_dtype, accumulate, M, N, K, activation, blocks, a_blocked, c_blocked, form, stream);
   }
 #define BH_PICK(FN, TILES, EXTRA, ...)                                             \
   do {                                                                              \
@@ -1461,8 +1462,8 @@ extern "C" int bh_gemm_bf16(const void* a, const void* w, void* c, int c_dtype, 
     } else {
       tiled_parts(M, N, K, layout, activation != 0, &parts, &each);
       const RidingNorm none = {};
-      if (activation) launch_tiled<true, true, float>(a, w, nullptr, M, N, K, 0, none, (float*)scratch, stream);
-      else launch_tiled<true, false, float>(a, w, nullptr, M, N, K, 0, none, (float*)scratch, stream);
+      if (activation) launch_tiled<true, true, float>(a, w, nullptr, M, N, K, 0, none, (float*)scratch, form, stream);
+      else launch_tiled<true, false, float>(a, w, nullptr, M, N, K, 0, none, (float*)scratch, form, stream);
       if (int status = bh_check_launch("gemm_tiled")) return status;
     }
     if (activation) { if (f32) BH_FINISH(true, float); else BH_FINISH(true, bf16_t); }
@@ -1474,20 +1475,20 @@ extern "C" int bh_gemm_bf16(const void* a, const void* w, void* c, int c_dtype, 
     const int pair_blocks = N / 16;
     const RowBlocks blocks = {a_block_rows, c_block_rows, behind_block_rows};
     if (activation) {
-      if (layout) BH_PICK(launch_skinny, true, 2, a, w, c, M, N, K, 0, pair_blocks, norm, blocks, stream);
-      else BH_PICK(launch_skinny, false, 2, a, w, c, M, N, K, 0, pair_blocks, norm, blocks, stream);
+      if (layout) BH_PICK(launch_skinny, true, 2, a, w, c, M, N, K, 0, pair_blocks, norm, blocks, form, stream);
+      else BH_PICK(launch_skinny, false, 2, a, w, c, M, N, K, 0, pair_blocks, norm, blocks, form, stream);
     } else {
-      if (layout) BH_PICK(launch_skinny, true, 1, a, w, c, M, N, K, accumulate, 0, norm, blocks, stream);
-      else BH_PICK(launch_skinny, false, 1, a, w, c, M, N, K, accumulate, 0, norm, blocks, stream);
+      if (layout) BH_PICK(launch_skinny, true, 1, a, w, c, M, N, K, accumulate, 0, norm, blocks, form, stream);
+      else BH_PICK(launch_skinny, false, 1, a, w, c, M, N, K, accumulate, 0, norm, blocks, form, stream);
     }
     return bh_check_launch("gemm_skinny");
   }
   if (activation) {
-    if (layout) BH_PICK(launch_tiled, true, true, a, w, c, M, N, K, 0, norm, nullptr, stream);
-    else BH_PICK(launch_tiled, false, true, a, w, c, M, N, K, 0, norm, nullptr, stream);
+    if (layout) BH_PICK(launch_tiled, true, true, a, w, c, M, N, K, 0, norm, nullptr, form, stream);
+    else BH_PICK(launch_tiled, false, true, a, w, c, M, N, K, 0, norm, nullptr, form, stream);
   } else {
-    if (layout) BH_PICK(launch_tiled, true, false, a, w, c, M, N, K, accumulate, norm, nullptr, stream);
-    else BH_PICK(launch_tiled, false, false, a, w, c, M, N, K, accumulate, norm, nullptr, stream);
+    if (layout) BH_PICK(launch_tiled, true, false, a, w, c, M, N, K, accumulate, norm, nullptr, form, stream);
+    else BH_PICK(launch_tiled, false, false, a, w, c, M, N, K, accumulate, norm, nullptr, form, stream);
   }
 #undef BH_PICK
   return bh_check_launch("gemm_tiled");

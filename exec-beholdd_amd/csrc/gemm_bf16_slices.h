@@ -11,8 +11,9 @@ int gemm_slices_parts(int M, int N, int K, int activation, int* slices_per_part)
 int gemm_slices_launch(const void* a, const void* w, float* sums, int M, int N, int K, int activation,
                        hipStream_t stream);
 // A SwiGLU with so many outputs that no parts are needed is finished by the kernel itself (gemm_slices_gated says
-// which): gated[M][N] = bfloat16(silu(a Wg^T) * (a Wu^T)), in blocks of gated_block_rows rows (0: rows), times the row
+// which): gated[M][N] = bfloat16(act(a Wg^T) * (a Wu^T)), act as `form` says, in blocks of gated_block_rows rows (0: rows), times the row
 // factors of a norm ahead when its partial sums are given.
 bool gemm_slices_gated(int M, int N, int K, int activation);
 int gemm_slices_launch_gated(const void* a, const void* w, void* gated, int gated_block_rows, int M, int N, int K,
-                             const float* ahead_ss, int ahead_blocks, float ahead_eps, hipStream_t stream);
+                             const float* ahead_ss, int ahead_blocks, float ahead_eps, GateForm form,
+                             hipStream_t stream);

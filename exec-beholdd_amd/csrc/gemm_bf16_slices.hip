@@ -59,7 +59,7 @@ constexpr int STAGE_K = 256;             // K is cut into parts at multiples of 
 // 640 5.50 -> 5.40 ms.
 // GATED: SwiGLU with all of K in one workgroup (one part): waves 0 to 3 own four blocks of gate rows, waves 4 to 7 the
 // blocks of up rows of the same outputs (N / 16 blocks further on); at the end the up waves hand their sums over
-// through LDS and the gate waves write bfloat16(silu(gate) * up), times the row factors of a norm ahead, into `gated`
+// through LDS and the gate waves write bfloat16(act(gate) * up), times the row factors of a norm ahead, into `gated`
 // (in blocks of gated_block_rows rows, or rows): no scratch memory and no finishing kernel.
 struct GatedOut {
   uint16_t* gated;        // [M][N] bfloat16
@@ -68,9 +68,8 @@ struct GatedOut {
   const float* ahead_ss;  // [M][ahead_blocks] partial sums of squares of the activations' rows, or null
   int ahead_blocks;
   float ahead_eps;
+  GateForm form;          // what stands on the gate
 };
-
-__device__ inline float silu_mul(float gate, float up) { return gate / (1.0f + expf(-gate)) * up; }
 
 template <int MB, int SC, int WAVES, bool GATED, bool DEEP = false>
 __global__ __launch_bounds__(64 * WAVES, GATED ? (WAVES + 3) / 4 : (MB > 4 || WAVES > 4) ? 2 : 4) void gemm_slices_kernel(const uint16_t* __restrict__ a,
@@ -213,8 +212,8 @@ __global__ __launch_bounds__(64 * WAVES, GATED ? (WAVES + 3) / 4 : (MB > 4 || WA
       uint32_t packed[2];
 #pragma unroll
       for (int i = 0; i < 2; ++i)
-        packed[i] = (uint32_t)f32_to_bf16_bits(silu_mul(acc[b][2 * i] * f, up[2 * i] * f)) |
-                    ((uint32_t)f32_to_bf16_bits(silu_mul(acc[b][2 * i + 1] * f, up[2 * i + 1] * f)) << 16);
+        packed[i] = (uint32_t)f32_to_bf16_bits(gate_mul(acc[b][2 * i] * f, up[2 * i] * f, out.form)) |
+                    ((uint32_t)f32_to_bf16_bits(gate_mul(acc[b][2 * i + 1] * f, up[2 * i + 1] * f, out.form)) << 16);
       uint32_t* at = reinterpret_cast<uint32_t*>(out.gated + bh_rows_index(out.gated_block_rows, m, n, out.N));
       at[0] = packed[0];
       at[1] = packed[1];
@@ -334,13 +333,13 @@ int gemm_slices_launch(const void* a, const void* w, float* sums, int M, int N, 
 }
 
 int gemm_slices_launch_gated(const void* a, const void* w, void* gated, int gated_block_rows, int M, int N, int K,
-                             const float* ahead_ss, int ahead_blocks, float ahead_eps, hipStream_t stream) {
+                             const float* ahead_ss, int ahead_blocks, float ahead_eps, GateForm form, hipStream_t stream) {
   BH_REQUIRE(gemm_slices_gated(M, N, K, 1), "gemm_slices: a SwiGLU of M=%d N=%d K=%d is not one this kernel finishes itself", M, N, K);
   BH_REQUIRE(((uintptr_t)a | (uintptr_t)w | (uintptr_t)gated) % 16 == 0, "gemm_slices: operands must be 16-byte aligned");
   BH_REQUIRE(!ahead_ss || (ahead_blocks > 0 && ahead_eps > 0.f), "gemm_slices: the norm ahead needs partial sums and an epsilon");
   constexpr int SC = GATED_CHUNKS;
   const int blocks_each = gated_blocks(M, N), WAVES = 2 * blocks_each;
-  const GatedOut out = {(uint16_t*)gated, gated_block_rows, N, ahead_ss, ahead_blocks, ahead_eps};
+  const GatedOut out = {(uint16_t*)gated, gated_block_rows, N, ahead_ss, ahead_blocks, ahead_eps, form};
   const dim3 grid((N / 16 + WAVES / 2 - 1) / (WAVES / 2)), block(64 * WAVES);
   const int stages = K / (64 * SC);
 #define BH_GATED(MB, NW) gemm_slices_kernel<MB, SC, NW, true, MB == 4><<<grid, block, 0, stream>>>((const uint16_t*)a, (const uint16_t*)w, nullptr, M, 2 * N, K, stages, out)

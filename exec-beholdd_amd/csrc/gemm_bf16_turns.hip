@@ -51,7 +51,6 @@ typedef uint32_t u32x2_t __attribute__((ext_vector_type(2)));
 namespace {
 
 __device__ inline bf16x8_t as_bf16x8(u32x4_t v) { return __builtin_bit_cast(bf16x8_t, v); }
-__device__ inline float silu_mul(float gate, float up) { return gate / (1.0f + expf(-gate)) * up; }
 
 // s_waitcnt immediates of gfx9: vmcnt in bits 3:0 and 15:14, expcnt 6:4, lgkmcnt 11:8.  Both wait for all
 // LDS reads; the first also until at most `vm` of the wave's global loads are still on their way.
@@ -96,7 +95,7 @@ __device__ inline void tile_of_workgroup(int n_tiles, int m_tiles, int* tile_n, 
   *tile_n = first_n + within / rows;
 }
 
-// MODE 0: bfloat16 output.  1: float32 output, optionally added to what is there.  2: SwiGLU, bfloat16 output
+// MODE 0: bfloat16 output.  1: float32 output, optionally added to what is there.  2: SwiGLU (the gate as `form` says), bfloat16 output
 // (N outputs; W has 2 N rows, gate rows then up rows; a wave's weight rows are the gate and the up rows of
 // the same outputs).  YB: blocks of 16 weight rows per wave.
 // A tile that would stick out of the matrix is moved back inside and stores only what it owns.
@@ -106,7 +105,7 @@ __device__ inline void tile_of_workgroup(int n_tiles, int m_tiles, int* tile_n, 
 template <int MODE, int YB>
 __global__ __launch_bounds__(512) void gemm_turns_kernel(const uint16_t* __restrict__ a, const uint16_t* __restrict__ w,
                                                       void* __restrict__ c, int M, int N, int K, int accumulate,
-                                                      int a_blocked, int c_blocked) {
+                                                      int a_blocked, int c_blocked, GateForm form) {
   constexpr int OUTS = MODE == 2 ? 16 * YB : 32 * YB;
   constexpr int CHUNKS = 16 + 2 * YB;
   constexpr int WL = YB / 2;   // W chunks per loading wave
@@ -233,8 +232,8 @@ __global__ __launch_bounds__(512) void gemm_turns_kernel(const uint16_t* __restr
         const int n = n0 + 8 * YB * g + 16 * y + 4 * (lane / 16);
         if (n < n_own) continue;
         u32x2_t packed;
-        packed[0] = f32_to_bf16_bits(silu_mul(acc[x][y][0], acc[x][y + YB / 2][0])) | ((uint32_t)f32_to_bf16_bits(silu_mul(acc[x][y][1], acc[x][y + YB / 2][1])) << 16);
-        packed[1] = f32_to_bf16_bits(silu_mul(acc[x][y][2], acc[x][y + YB / 2][2])) | ((uint32_t)f32_to_bf16_bits(silu_mul(acc[x][y][3], acc[x][y + YB / 2][3])) << 16);
+        packed[0] = f32_to_bf16_bits(gate_mul(acc[x][y][0], acc[x][y + YB / 2][0], form)) | ((uint32_t)f32_to_bf16_bits(gate_mul(acc[x][y][1], acc[x][y + YB / 2][1], form)) << 16);
+        packed[1] = f32_to_bf16_bits(gate_mul(acc[x][y][2], acc[x][y + YB / 2][2], form)) | ((uint32_t)f32_to_bf16_bits(gate_mul(acc[x][y][3], acc[x][y + YB / 2][3], form)) << 16);
         *reinterpret_cast<u32x2_t*>(out + (c_blocked ? (size_t)bh_blocked_index(row, n, N) : (size_t)row * N + n)) = packed;
       }
     }
@@ -270,11 +269,11 @@ __global__ __launch_bounds__(512) void gemm_turns_kernel(const uint16_t* __restr
 
 template <int MODE>
 void launch(const void* a, const void* w, void* c, int blocks, int M, int N, int K, int accumulate, int a_blocked,
-            int c_blocked, hipStream_t stream, int parts = 1) {
+            int c_blocked, GateForm form, hipStream_t stream, int parts = 1) {
   const int outs = (MODE == 2 ? 16 : 32) * blocks;
   dim3 grid(((N + outs - 1) / outs) * ((M + 255) / 256), parts);
 #define BH_TURNS(YB) \
-  gemm_turns_kernel<MODE, YB><<<grid, 512, 0, stream>>>((const uint16_t*)a, (const uint16_t*)w, c, M, N, K, accumulate, a_blocked, c_blocked)
+  gemm_turns_kernel<MODE, YB><<<grid, 512, 0, stream>>>((const uint16_t*)a, (const uint16_t*)w, c, M, N, K, accumulate, a_blocked, c_blocked, form)
   if (blocks == 8) BH_TURNS(8);
   else if (blocks == 6) BH_TURNS(6);
   else BH_TURNS(4);
@@ -373,12 +372,12 @@ int gemm_turns_launch_parts(const void* a, const void* w, float* sums, int M, in
   BH_REQUIRE(parts >= 1 && K % (128 * parts) == 0 && gemm_turns_can(M, N, K / parts, 1, 0, pb),
              "gemm_turns: M=%d N=%d K=%d cannot be multiplied in %d parts of K", M, N, K, parts);
   BH_REQUIRE(((uintptr_t)a | (uintptr_t)w | (uintptr_t)sums) % 16 == 0, "gemm_turns: operands must be 16-byte aligned");
-  launch<1>(a, w, sums, pb, M, N, K, 0, a_blocked, 0, stream, parts);
+  launch<1>(a, w, sums, pb, M, N, K, 0, a_blocked, 0, GateForm{}, stream, parts);
   return bh_check_launch("gemm_turns");
 }
 
 int gemm_turns_launch(const void* a, const void* w, void* c, int c_dtype, int accumulate, int M, int N, int K,
-                      int activation, int blocks, int a_blocked, int c_blocked, hipStream_t stream) {
+                      int activation, int blocks, int a_blocked, int c_blocked, GateForm form, hipStream_t stream) {
   BH_REQUIRE(gemm_turns_can(M, N, K, 1, activation, blocks),
              "gemm_turns: a product of M=%d N=%d K=%d with %d blocks per wave is not one this kernel takes "
              "(M >= 256, K a multiple of 128, N a multiple of 16 and at least a tile)", M, N, K, blocks);
@@ -388,16 +387,16 @@ int gemm_turns_launch(const void* a, const void* w, void* c, int c_dtype, int ac
   BH_REQUIRE(((uintptr_t)a | (uintptr_t)w | (uintptr_t)c) % 16 == 0 && (c_dtype == BH_F32 || N % 4 == 0),
              "gemm_turns: operands and output must be 16-byte aligned");
   BH_REQUIRE(!c_blocked || (activation && N % 32 == 0), "gemm_turns: only SwiGLU writes its output in blocks, and N=%d must be a multiple of 32", N);
-  if (activation) launch<2>(a, w, c, blocks, M, N, K, 0, a_blocked, c_blocked, stream);
-  else if (c_dtype == BH_F32) launch<1>(a, w, c, blocks, M, N, K, accumulate, a_blocked, 0, stream);
-  else launch<0>(a, w, c, blocks, M, N, K, 0, a_blocked, 0, stream);
+  if (activation) launch<2>(a, w, c, blocks, M, N, K, 0, a_blocked, c_blocked, form, stream);
+  else if (c_dtype == BH_F32) launch<1>(a, w, c, blocks, M, N, K, accumulate, a_blocked, 0, form, stream);
+  else launch<0>(a, w, c, blocks, M, N, K, 0, a_blocked, 0, form, stream);
   return bh_check_launch("gemm_turns");
 }
 
 // For tests and measurements: the kernel at a given tile width, whatever gemm_turns_blocks would choose.
 extern "C" int bh_gemm_bf16_turns(const void* a, const void* w, void* c, int c_dtype, int accumulate, int M, int N,
                                   int K, int activation, int blocks, int a_blocked, int c_blocked, hipStream_t stream) {
-  return gemm_turns_launch(a, w, c, c_dtype, accumulate, M, N, K, activation, blocks, a_blocked, c_blocked, stream);
+  return gemm_turns_launch(a, w, c, c_dtype, accumulate, M, N, K, activation != 0, blocks, a_blocked, c_blocked, bh_gate_form(activation), stream);
 }
 extern "C" int bh_gemm_bf16_turns_blocks(int M, int N, int K, int layout, int activation) {
   return gemm_turns_blocks(M, N, K, layout, activation);

@@ -838,29 +838,30 @@ extern "C" int bh_attention_generic(const void* q, void* out, int dtype, const v
 }
 
 // ---- SwiGLU ---------------------------------------------------------------------------------
-// out[r, i] = silu(gu[r, i]) * gu[r, F + i], silu(x) = x / (1 + exp(-x)).
+// out[r, i] = silu(gu[r, i]) * gu[r, F + i], silu(x) = x / (1 + exp(-x)), or the tanh form of GELU in its place (BhGate).
 
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int F, size_t total) {
+__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int F, size_t total, GateForm form) {
   const size_t at = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (at >= total) return;
   const size_t r = at / F;
   const int i = (int)(at % F);
   const float g = to_f32(gu[r * 2 * F + i]);
   const float u = to_f32(gu[r * 2 * F + F + i]);
-  out[at] = from_f32<T>(g / (1.0f + expf(-g)) * u);
+  out[at] = from_f32<T>(gate_mul(g, u, form));
 }
 
-extern "C" int bh_swiglu(const void* gu, void* out, int dtype, int n_rows, int F, hipStream_t stream) {
+extern "C" int bh_swiglu(const void* gu, void* out, int dtype, int n_rows, int F, int gate, hipStream_t stream) {
+  BH_REQUIRE(gate == BH_GATE_SILU || gate == BH_GATE_GELU_TANH, "swiglu: unknown gate %d", gate);
   BH_REQUIRE(n_rows > 0 && F > 0, "swiglu: sizes must be positive");
   const size_t total = (size_t)n_rows * F;
   const size_t blocks = (total + 255) / 256;
   BH_REQUIRE(blocks <= 2147483647u, "swiglu: too many elements");
   dim3 grid((unsigned)blocks), block(256);
   if (dtype == BH_F32)
-    swiglu_kernel<float><<<grid, block, 0, stream>>>((const float*)gu, (float*)out, F, total);
+    swiglu_kernel<float><<<grid, block, 0, stream>>>((const float*)gu, (float*)out, F, total, bh_gate_form(gate));
   else if (dtype == BH_BF16)
-    swiglu_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, F, total);
+    swiglu_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, F, total, bh_gate_form(gate));
   else
     return bh_fail("swiglu: unknown dtype %d", dtype);
   return bh_check_launch("swiglu");

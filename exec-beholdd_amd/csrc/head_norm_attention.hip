@@ -7,6 +7,9 @@
 //                          head of q and k turned by position * freq[i];  q into a matrix of heads of `pad` dimensions, k and v
 //                          into the cache pages of (sequence, position) as heads of `pad` (zeros beyond dim and vdim), so that
 //                          keys of one size and values of another go through kernels that know one head size.
+//                          `unit_norm`: that norm without weights (a turn keeps a head's length, so it does not matter which of
+//                          the two comes first).  `values_are_keys`: the row holds no v, a head's value is its key as it stands
+//                          there, ahead of norm and turn; one wave then writes both.
 // Sums, statistics, angles, cosines and sines are float32; the angle is the float32 product position * freq[i].
 #include "common.h"
 
@@ -21,7 +24,7 @@ __global__ __launch_bounds__(HN_WAVES * BH_WAVE) void head_norm_rope_write_kerne
     const float* __restrict__ wk, float eps, const float* __restrict__ freq, int turned, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ row_seq, T* __restrict__ q_out, T* __restrict__ k_pages, T* __restrict__ v_pages,
     const int32_t* __restrict__ page_table, int table_stride, int H, int G, int dim, int vdim, int pad, int kv_order, int write,
-    int per_group, int neighbours, float magnitude) {
+    int per_group, int neighbours, float magnitude, int unit_norm, int values_are_keys) {
   extern __shared__ float lds[];      // the cosines and sines of the row's turned pairs, then a head of `dim` floats a wave
   const int row = blockIdx.x, wave = threadIdx.x / BH_WAVE, lane = threadIdx.x % BH_WAVE;
   const int half = turned / 2;
@@ -40,7 +43,7 @@ __global__ __launch_bounds__(HN_WAVES * BH_WAVE) void head_norm_rope_write_kerne
   int page = 0;
   const int token = pos % BH_PAGE;
   if (write) page = page_table[(size_t)row_seq[row] * table_stride + pos / BH_PAGE];
-  const int heads = write ? H + 2 * G : H;
+  const int heads = write ? (values_are_keys ? H + G : H + 2 * G) : H;
   const int stretch_end = ((int)blockIdx.y + 1) * per_group < heads ? ((int)blockIdx.y + 1) * per_group : heads;
   for (int unit = blockIdx.y * per_group + wave; unit < stretch_end; unit += HN_WAVES) {
     if (unit >= H + G) {      // a head of values: the bias, and zeros beyond vdim
@@ -62,11 +65,15 @@ __global__ __launch_bounds__(HN_WAVES * BH_WAVE) void head_norm_rope_write_kerne
       ss += v * v;
     }
     ss = wave_sum(ss);
-    const float inv = w ? 1.0f / sqrtf(ss / (float)dim + eps) : 1.0f;
+    const float inv = w || unit_norm ? 1.0f / sqrtf(ss / (float)dim + eps) : 1.0f;
     // (a wave's lanes run together: what the lanes wrote above is there for all of them below)
     __builtin_amdgcn_wave_barrier();
     T* keys = is_key ? k_pages + ((size_t)page * G + head) * BH_PAGE * pad : nullptr;
     T* queries = q_out + ((size_t)row * H + head) * pad;
+    if (is_key && values_are_keys) {
+      T* values = v_pages + ((size_t)page * G + head) * BH_PAGE * pad;
+      for (int i = lane; i < pad; i += BH_WAVE) values[bh_value_index(kv_order, token, i, pad)] = from_f32<T>(i < dim ? mine[i] : 0.f);
+    }
     for (int i = lane; i < pad; i += BH_WAVE) {
       float y = 0.f;
       if (i < dim) {
@@ -96,18 +103,20 @@ extern "C" int bh_head_norm_rope_write(const void* proj, int dtype, int row_stri
                                        const float* wk, float eps, const float* freq, int turned, const int32_t* positions,
                                        const int32_t* row_seq, void* q_out, void* k_pages, void* v_pages, const int32_t* page_table,
                                        int table_stride, int n_rows, int H, int G, int dim, int vdim, int pad, int kv_order, int write,
-                                       int neighbours, float magnitude, hipStream_t stream) {
+                                       int neighbours, float magnitude, int unit_norm, int values_are_keys, hipStream_t stream) {
   BH_REQUIRE(n_rows > 0 && H > 0 && G > 0 && dim > 0 && vdim > 0, "head_norm_rope_write: sizes must be positive");
   BH_REQUIRE(pad >= dim && pad >= vdim, "head_norm_rope_write: heads of %d do not hold keys of %d and values of %d", pad, dim, vdim);
   BH_REQUIRE(turned >= 0 && turned % 2 == 0 && turned <= dim, "head_norm_rope_write: %d turned dimensions of %d", turned, dim);
   BH_REQUIRE(turned == 0 || freq != nullptr, "head_norm_rope_write: a rotation needs its frequencies");
   BH_REQUIRE((wq == nullptr) == (wk == nullptr), "head_norm_rope_write: give both norm weights or neither");
-  BH_REQUIRE(first >= 0 && first + (H + G) * dim + G * vdim <= row_stride, "head_norm_rope_write: q, k and v lie outside a row of %d", row_stride);
+  BH_REQUIRE(!unit_norm || wq == nullptr, "head_norm_rope_write: a norm without weights has none");
+  BH_REQUIRE(!values_are_keys || vdim == dim, "head_norm_rope_write: values that are keys of %d have that size, not %d", dim, vdim);
+  BH_REQUIRE(first >= 0 && first + (H + G) * dim + (values_are_keys ? 0 : G * vdim) <= row_stride, "head_norm_rope_write: q, k and v lie outside a row of %d", row_stride);
   BH_REQUIRE(kv_order == BH_KV_ROWS || (kv_order == BH_KV_PIECES && pad % 32 == 0),
              "head_norm_rope_write: cache order %d does not exist for head size %d", kv_order, pad);
   const size_t lds = (size_t)(turned + HN_WAVES * dim) * sizeof(float);
   BH_REQUIRE(lds <= 48 * 1024, "head_norm_rope_write: heads of %d dimensions do not fit the local memory", dim);
-  const int heads = write ? H + 2 * G : H;
+  const int heads = write ? (values_are_keys ? H + G : H + 2 * G) : H;
   const int per_group = n_rows >= 4 * bh_compute_units() ? 4 * HN_WAVES : HN_WAVES;      // many rows fill the chip by themselves
   const dim3 grid(n_rows, (heads + per_group - 1) / per_group);
   BH_REQUIRE(grid.y <= 65535, "head_norm_rope_write: too many heads");
@@ -115,7 +124,7 @@ extern "C" int bh_head_norm_rope_write(const void* proj, int dtype, int row_stri
   head_norm_rope_write_kernel<T><<<grid, HN_WAVES * BH_WAVE, lds, stream>>>((const T*)proj, row_stride, first, bias, wq, wk, eps, freq, \
                                                                            turned, positions, row_seq, (T*)q_out, (T*)k_pages,    \
                                                                            (T*)v_pages, page_table, table_stride, H, G, dim, vdim, \
-                                                                           pad, kv_order, write, per_group, neighbours, magnitude)
+                                                                           pad, kv_order, write, per_group, neighbours, magnitude, unit_norm, values_are_keys)
   if (dtype == BH_F32) BH_HN(float);
   else if (dtype == BH_BF16) BH_HN(bf16_t);
   else return bh_fail("head_norm_rope_write: unknown dtype %d", dtype);

@@ -1,6 +1,7 @@
 // Small row-wise operations on the float32 residual and on logits:
 //   layernorm        (x - mean) / sqrt(var + eps) * w + b per row, optional row gather, rows or blocks of rows out
 //   sum_layernorm    h <- layernorm(alpha h + y) per row in place, and the same rounded for the product that reads it next
+//   add_rmsnorm      h <- h + y / sqrt(mean(y^2) + eps) * w per row in place, and the same rounded for the product that reads it next
 //   gelu_tanh        out = gelu(x), tanh form, elementwise into rows or blocks of rows
 //   cast_concat      [a | b] per row from float32 into the activation type (b optional): the input of a product
 //   softcap          x <- cap * tanh(x / cap) in place
@@ -148,6 +149,84 @@ extern "C" int bh_sum_layernorm(float* h, const float* y, float alpha, const flo
   else
     return bh_fail("sum_layernorm: unknown dtype %d", out_dtype);
   return bh_check_launch("sum_layernorm");
+}
+
+// h <- h + y / sqrt(mean(y^2) + eps) * w: the norm of what a sublayer gave, added to the residual.  One workgroup a row; a thread
+// keeps its PER elements of y and h in registers (PER 0: rows longer than that are read twice).  w: float32 or bfloat16.
+template <typename TO, typename TW, int PER, int THREADS>
+__global__ __launch_bounds__(THREADS) void add_rmsnorm_kernel(float* __restrict__ h, const float* __restrict__ y, const TW* __restrict__ w,
+                                                              TO* __restrict__ rounded, int width, float eps, int out_block_rows) {
+  __shared__ float scratch[THREADS / BH_WAVE];
+  const int r = blockIdx.x;
+  float* row = h + (size_t)r * width;
+  const float* add = y + (size_t)r * width;
+  constexpr int HELD = PER ? PER : 1;
+  float held[HELD], before[HELD];
+  float ss = 0.f;
+  if constexpr (PER > 0) {
+#pragma unroll
+    for (int k = 0; k < PER; ++k) {
+      const int i = threadIdx.x + k * THREADS;
+      held[k] = i < width ? add[i] : 0.f;
+      before[k] = i < width ? row[i] : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < PER; ++k) ss += held[k] * held[k];
+  } else {
+    for (int i = threadIdx.x; i < width; i += THREADS) ss += add[i] * add[i];
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)width + eps);
+  auto finish = [&](int i, float value, float old) {
+    const float v = old + value * inv * to_f32(w[i]);
+    row[i] = v;
+    if (rounded) rounded[bh_rows_index(out_block_rows, r, i, width)] = from_f32<TO>(v);
+  };
+  if constexpr (PER > 0) {
+#pragma unroll
+    for (int k = 0; k < PER; ++k) {
+      const int i = threadIdx.x + k * THREADS;
+      if (i < width) finish(i, held[k], before[k]);
+    }
+  } else {
+    for (int i = threadIdx.x; i < width; i += THREADS) finish(i, add[i], row[i]);
+  }
+}
+
+template <typename TO, typename TW>
+static void add_rmsnorm_launch(float* h, const float* y, const TW* w, TO* rounded, int n_rows, int width, float eps, int out_block_rows,
+                               hipStream_t stream) {
+#define BH_AN(PER, THREADS) add_rmsnorm_kernel<TO, TW, PER, THREADS><<<n_rows, THREADS, 0, stream>>>(h, y, w, rounded, width, eps, out_block_rows)
+  if (n_rows <= 64 && width > 1024 && width <= 1024 * 8) {      // few rows: a row on sixteen waves, a few elements a thread
+    if (width <= 1024 * 4) BH_AN(4, 1024);
+    else BH_AN(8, 1024);
+  } else if (width <= 256 * 4) {
+    BH_AN(4, 256);
+  } else if (width <= 256 * 16) {
+    BH_AN(16, 256);
+  } else {
+    BH_AN(0, 256);
+  }
+#undef BH_AN
+}
+
+extern "C" int bh_add_rmsnorm(float* h, const float* y, const void* w, int w_dtype, void* rounded, int out_dtype, int n_rows, int width,
+                              float eps, int out_block_rows, hipStream_t stream) {
+  BH_REQUIRE(n_rows > 0 && width > 0, "add_rmsnorm: sizes must be positive");
+  BH_REQUIRE(h != y, "add_rmsnorm: the sublayer's result stands apart from the residual");
+  BH_REQUIRE(w_dtype == BH_F32 || w_dtype == BH_BF16, "add_rmsnorm: unknown weight dtype %d", w_dtype);
+  BH_REQUIRE(rounded == nullptr || out_dtype == BH_F32 || out_dtype == BH_BF16, "add_rmsnorm: unknown dtype %d", out_dtype);
+  BH_REQUIRE(out_block_rows == 0 || (rounded && (out_block_rows == 8 || out_block_rows == 16) && width % 32 == 0 && out_dtype == BH_BF16),
+             "add_rmsnorm: rows in blocks of %d of width %d are not written", out_block_rows, width);
+#define BH_ADD(TO, TW) add_rmsnorm_launch<TO, TW>(h, y, (const TW*)w, (TO*)rounded, n_rows, width, eps, out_block_rows, stream)
+  if (rounded == nullptr || out_dtype == BH_F32) {
+    if (w_dtype == BH_F32) BH_ADD(float, float);
+    else BH_ADD(float, bf16_t);
+  } else {
+    if (w_dtype == BH_F32) BH_ADD(bf16_t, float);
+    else BH_ADD(bf16_t, bf16_t);
+  }
+#undef BH_ADD
+  return bh_check_launch("add_rmsnorm");
 }
 
 template <typename TO>

@@ -144,7 +144,7 @@ class KernelSizes:
             "bh_gemm_bf16_bare_parts": [i, i, i, i],
             "bh_gemm_bf16_bare": [p, p, p, i, i, i, i, i, p],
             "bh_attention_generic": [p, p, i, p, p, p, i, p, p, i, i, i, i, f, i, i, p, p],
-            "bh_swiglu": [p, p, i, i, i, p],
+            "bh_swiglu": [p, p, i, i, i, i, p],
             "bh_sample": [p, p, p, p, p, p, p, p, i, i, p],
             "bh_sample_scratch": [i, i],
             "bh_sample_draw_scratch": [i, i],
@@ -175,9 +175,10 @@ class KernelSizes:
             "bh_rotate_heads": [p, ctypes.c_long, i, i, p, ctypes.c_long, i, i, i, p, i, p, i, i, i, p],
             "bh_layernorm": [p, p, p, p, p, i, i, i, f, i, p],
             "bh_cast_concat": [p, p, p, i, i, i, i, p],
+            "bh_add_rmsnorm": [p, p, p, i, p, i, i, i, f, i, p],
             "bh_sum_layernorm": [p, p, f, p, p, p, i, i, i, f, i, p],
             "bh_gelu_tanh": [p, p, i, i, i, i, p],
-            "bh_head_norm_rope_write": [p, i, i, i, p, p, p, f, p, i, p, p, p, p, p, p, i, i, i, i, i, i, i, i, i, i, f, p],
+            "bh_head_norm_rope_write": [p, i, i, i, p, p, p, f, p, i, p, p, p, p, p, p, i, i, i, i, i, i, i, i, i, i, f, i, i, p],
             "bh_mlstm_gates": [p, p, f, p, ctypes.c_long, i, p, p, p, i, i, p],
             "bh_mlstm_scan": [p, i, i, i, i, i, p, p, ctypes.c_long, p, p, p, i, i, i, i, p],
             "bh_mlstm_finish": [p, p, p, i, i, i, p, f, p, i, i, i, i, p],
@@ -191,9 +192,9 @@ class KernelSizes:
             "bh_gate_heads": [p, i, i, p, i, i, p, i, i, i, i, i, p],
             "bh_ssm_scan": [p, i, p, i, i, i, p, p, p, p, ctypes.c_long, p, p, p, i, i, i, i, i, p],
             "bh_gated_group_rmsnorm": [p, p, i, i, i, p, f, p, i, i, i, i, i, p],
-            "bh_route_top_k": [p, p, p, p, i, i, i, i, p],
-            "bh_experts_gate_up": [p, i, p, p, p, i, i, i, i, f, f, f, p, p],
-            "bh_experts_down": [p, i, p, p, p, p, i, i, i, i, p],
+            "bh_route_top_k": [p, p, p, p, p, i, i, i, i, p],
+            "bh_experts_gate_up": [p, i, p, p, p, i, i, i, i, i, f, f, f, p, p],
+            "bh_experts_down": [p, i, p, p, p, p, p, i, i, i, i, i, i, p],
             "bh_clamped_glu": [p, i, p, i, i, f, f, i, f, p],
             "bh_conv_norm_rope_write": [p, i, i, i, p, i, p, ctypes.c_long, p, p, p, p, f, p, i, p, p, p, p, p, p, i, i, i, i, i, i, i, i, i, p],
             "bh_ssm_scan_fast": [p, i, p, i, i, i, p, p, p, p, ctypes.c_long, p, p, p, p, p, p, i, i, i, i, i, i, i, p],
@@ -208,7 +209,7 @@ class KernelSizes:
             "bh_gla_chunk_rows": [i, i, i, i, i],
             "bh_slice_rmsnorm": [p, i, i, i, p, f, p, i, i, i, p],
             "bh_weighted_sum": [p, p, f, p, f, ctypes.c_long, p],
-            "bh_experts_combine": [p, p, p, p, i, i, i, p],
+            "bh_experts_combine": [p, p, p, p, p, i, p, i, i, i, i, i, p],
         }
         for name, argtypes in table.items():
             function = getattr(lib, name)
@@ -457,7 +458,9 @@ class HipKernels(KernelSizes):
             return PackedWeight(data, rows, cols)
         return w
 
-    def _gemm_fast(self, a, w, out, accumulate, activation, then_norm=None):
+    GATES = {"silu": 1, "gelu_tanh": 2}      # what may stand on the gate of a gated feed-forward (csrc/common.h: BhGate)
+
+    def _gemm_fast(self, a, w, out, accumulate, activation, then_norm=None, gate=1):
         """Launch the matrix-core product if it takes these operands; say whether it did, and with
         what prepared norm output (None if `then_norm` was not asked for or cannot ride on this product)."""
         fast = self.lib.bh_gemm_bf16
@@ -516,7 +519,7 @@ class HipKernels(KernelSizes):
             scratch = torch.empty(scratch_bytes // 4, dtype=torch.float32, device=self.device)
         self._check(fast(
             self._ptr(a_rows, "gemm a"), self._ptr(w.data if packed else w, "gemm w"), self._ptr(out, "gemm out"),
-            _code(out, "gemm out"), int(bool(accumulate)), m, n, k, int(packed), int(activation),
+            _code(out, "gemm out"), int(bool(accumulate)), m, n, k, int(packed), int(gate if activation else 0),
             self._ptr(ahead.ss, "norm sums") if ahead is not None else None,
             ahead.ss.shape[1] if ahead is not None else 0, ahead.eps if ahead is not None else 0.0,
             self._ptr(then_norm.weight, "norm weight") if behind is not None else None,
@@ -615,9 +618,9 @@ class HipKernels(KernelSizes):
         self.rmsnorm(prepared.source, prepared.weight, prepared.eps, out)
         return out
 
-    def gemm_swiglu(self, a, w, out):
+    def gemm_swiglu(self, a, w, out, gate="silu"):
         """out[M, F] = silu(a @ w[:F]^T) * (a @ w[F:]^T) for w [2F, K] = gate rows, then up rows; `a` may
-        be NormedRows."""
+        be NormedRows.  `gate`: "silu", or "gelu_tanh" for GELU's tanh form in its place."""
         if a.dim() != 2 or w.dim() != 2 or out.dim() != 2:
             raise KernelError("gemm_swiglu: operands must be matrices")
         m, k = a.shape
@@ -627,18 +630,18 @@ class HipKernels(KernelSizes):
                               "do not fit")
         if isinstance(a, NormedRows) and width % 16 == 0 and not self._takes_norm(a, w, width, 1):
             a = self._run_norm(a)
-        if self._gemm_fast(a, w, out, False, 1)[0]:
+        if self._gemm_fast(a, w, out, False, 1, gate=self.GATES[gate])[0]:
             return
         if isinstance(out, BlockedRows):      # this product writes rows, or not these blocks: regroup them afterwards
             rows_out = torch.empty((m, width), dtype=out.dtype, device=self.device)
-            self.gemm_swiglu(a, w, rows_out)
+            self.gemm_swiglu(a, w, rows_out, gate)
             self.to_blocked(rows_out, out)
             return
         if isinstance(a, BlockedRows):
             a = self.from_blocked(a)
         both = torch.empty((m, 2 * width), dtype=a.dtype, device=self.device)
         self.gemm(a, w, both)
-        self.swiglu(both, out)
+        self.swiglu(both, out, gate)
 
     def qk_norm_rope_cache(self, qkv, q_out, q_weight, k_weight, eps, cos, sin, positions, row_seq,
                            k_pages, v_pages, page_table, n_heads, n_kv_heads, head_dim, write_kv, max_position):
@@ -1059,6 +1062,18 @@ class HipKernels(KernelSizes):
             self._ptr(rounded, "sum_layernorm rounded", None, True), _code(rounded, "sum_layernorm rounded") if rounded is not None else F32,
             n_rows, width, float(eps), _block_rows(rounded) if rounded is not None else 0, self._stream()))
 
+    def add_rmsnorm(self, hidden, y, weight, eps, rounded=None):
+        """hidden[r] <- hidden[r] + y[r] / sqrt(mean(y[r]^2) + eps) * weight in place (hidden and y f32, weight f32 or bfloat16);
+        `rounded` [n, D], if given, takes the same in its own type, in rows or blocks of rows."""
+        n_rows, width = hidden.shape
+        if tuple(y.shape) != (n_rows, width) or weight.shape != (width,) or (rounded is not None and tuple(rounded.shape) != (n_rows, width)):
+            raise KernelError(f"add_rmsnorm: shapes hidden {tuple(hidden.shape)}, y {tuple(y.shape)} do not fit")
+        self._check(self.lib.bh_add_rmsnorm(
+            self._ptr(hidden, "add_rmsnorm hidden", (torch.float32,)), self._ptr(y, "add_rmsnorm y", (torch.float32,)),
+            self._ptr(weight, "add_rmsnorm weight"), _code(weight, "add_rmsnorm weight"), self._ptr(rounded, "add_rmsnorm rounded", None, True),
+            _code(rounded, "add_rmsnorm rounded") if rounded is not None else F32, n_rows, width, float(eps),
+            _block_rows(rounded) if rounded is not None else 0, self._stream()))
+
     def gelu_tanh(self, x, out=None):
         """out <- x/2 (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))); in place without `out`, which may be `BlockedRows`."""
         out = x if out is None else out
@@ -1069,14 +1084,15 @@ class HipKernels(KernelSizes):
 
     def head_norm_rope_write(self, proj, first, bias, q_weight, k_weight, eps, freq, turned, positions, row_seq, q_out, k_pages,
                              v_pages, page_table, n_heads, n_kv_heads, dim, vdim, pad, write_kv, neighbours=False,
-                             magnitude=1.0):
+                             magnitude=1.0, unit_norm=False, values_are_keys=False):
         """From column `first` of every row of `proj` [n, P]: q (H heads of dim), k (G of dim), v (G of vdim), plus `bias` (f32
         over those channels, or None); every head of q and k normed by its own root mean square times q_weight / k_weight
         (f32 [dim], both or None); dimensions i and i + turned/2 of every head of q and k turned by position * freq[i];
         (`neighbours`: dimensions 2i and 2i + 1 instead; `magnitude` multiplies every cosine and sine);
-        q -> q_out [n, H pad], k and v into the cache pages as heads of `pad` (see csrc/head_norm_attention.hip)."""
+        q -> q_out [n, H pad], k and v into the cache pages as heads of `pad` (see csrc/head_norm_attention.hip).
+        `unit_norm`: that norm without weights; `values_are_keys`: the rows hold no v, a head's value is its k, not normed or turned."""
         n_rows = proj.shape[0]
-        channels = (n_heads + n_kv_heads) * dim + n_kv_heads * vdim
+        channels = (n_heads + n_kv_heads) * dim + (0 if values_are_keys else n_kv_heads * vdim)
         if tuple(q_out.shape) != (n_rows, n_heads * pad) or q_out.dtype != proj.dtype or first < 0 or first + channels > proj.shape[1]:
             raise KernelError(f"head_norm_rope_write: shapes proj {tuple(proj.shape)}, q_out {tuple(q_out.shape)} do not fit")
         if (q_weight is None) != (k_weight is None) or (q_weight is not None and (q_weight.shape != (dim,) or k_weight.shape != (dim,))):
@@ -1095,7 +1111,8 @@ class HipKernels(KernelSizes):
             self._ptr(freq, "frequencies", f32, True), int(turned), self._ptr(positions, "positions", i32),
             self._ptr(row_seq, "row_seq", i32), self._ptr(q_out, "q_out"), self._ptr(k_pages, "k_pages"), self._ptr(v_pages, "v_pages"),
             self._ptr(page_table, "page_table", i32), page_table.shape[1], n_rows, n_heads, n_kv_heads, dim, vdim, pad,
-            self.kv_order(k_pages.dtype, pad), int(bool(write_kv)), int(bool(neighbours)), float(magnitude), self._stream()))
+            self.kv_order(k_pages.dtype, pad), int(bool(write_kv)), int(bool(neighbours)), float(magnitude), int(bool(unit_norm)),
+            int(bool(values_are_keys)), self._stream()))
 
     # ---- a matrix memory with exponential gates, as a recurrence over a float32 state ----
     MLSTM_BESIDE = 4      # floats a row and head beside the read-out: a_t, b_t, m_t, n_t . q_t
@@ -1377,24 +1394,29 @@ class HipKernels(KernelSizes):
             self._ptr(out, "gated_group_rmsnorm out"), n_rows, width, int(groups), _block_rows(out), int(bool(gate_after)), self._stream()))
 
     # ---- routed experts ----
-    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax"):
+    SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_all": 2}
+
+    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax", correction=None):
         """chosen[r] = the `top` largest of logits[r] + bias (largest first, ties to the lower index), weights[r] = softmax over
         those alone; logits f32 [n, E], chosen int32 [n, top], weights f32 [n, top].
-        `scoring` "sigmoid": weights[r] = the sigmoid of every chosen logit, each for itself."""
-        if scoring not in ("softmax", "sigmoid"):
-            raise KernelError(f"route_top_k: scoring is 'softmax' or 'sigmoid', got {scoring!r}")
+        `scoring` "sigmoid": weights[r] = the sigmoid of every chosen logit, each for itself.  "softmax_all": weights[r] = the
+        chosen ones' shares of the softmax over all E, and the choice goes by share + `correction` (f32 [E])."""
+        if scoring not in self.SCORINGS or (correction is not None and scoring != "softmax_all"):
+            raise KernelError(f"route_top_k: scoring is one of {sorted(self.SCORINGS)} (a correction goes with 'softmax_all'), got {scoring!r}")
         n_rows, experts = logits.shape
         top = chosen.shape[1]
-        if chosen.shape != (n_rows, top) or weights.shape != (n_rows, top) or (bias is not None and bias.shape != (experts,)):
+        if chosen.shape != (n_rows, top) or weights.shape != (n_rows, top) or any(
+                t is not None and t.shape != (experts,) for t in (bias, correction)):
             raise KernelError(f"route_top_k: shapes logits {tuple(logits.shape)}, chosen {tuple(chosen.shape)} do not fit")
         self._check(self.lib.bh_route_top_k(
             self._ptr(logits, "router logits", (torch.float32,)), self._ptr(bias, "router bias", (torch.float32,), True),
-            self._ptr(chosen, "chosen", (torch.int32,)), self._ptr(weights, "route weights", (torch.float32,)), n_rows, experts, top,
-            int(scoring == "sigmoid"), self._stream()))
+            self._ptr(correction, "router correction", (torch.float32,), True), self._ptr(chosen, "chosen", (torch.int32,)), self._ptr(weights, "route weights", (torch.float32,)), n_rows, experts, top,
+            self.SCORINGS[scoring], self._stream()))
 
     def experts_gate_up(self, h, chosen, w_gate_up, inner, limit, alpha, shift=1.0, in_weights=None):
         """inner[r * top + j] = act(Wg_e h[r], Wu_e h[r]) for e = chosen[r, j]; w_gate_up [E, 2 ff, K] (gate rows, then up rows).
-        `in_weights` float32 [n, top]: a pair's weight multiplies the expert's input (its gate and up sums)."""
+        `in_weights` float32 [n, top]: a pair's weight multiplies the expert's input (its gate and up sums).  Pairs whose expert
+        is numbered E or higher are left out."""
         n_rows, k = h.shape
         top = chosen.shape[1]
         experts, twice, k_w = w_gate_up.shape
@@ -1404,20 +1426,27 @@ class HipKernels(KernelSizes):
             raise KernelError(f"experts_gate_up: shapes h {tuple(h.shape)}, weights {tuple(w_gate_up.shape)}, inner {tuple(inner.shape)} do not fit")
         self._check(self.lib.bh_experts_gate_up(
             self._ptr(h, "experts h"), _code(h, "experts h"), self._ptr(chosen, "chosen", (torch.int32,)), self._ptr(w_gate_up, "expert gate/up"),
-            self._ptr(inner, "experts inner"), n_rows, top, k, ff, float(limit), float(alpha), float(shift),
+            self._ptr(inner, "experts inner"), n_rows, top, experts, k, ff, float(limit), float(alpha), float(shift),
             self._ptr(in_weights, "pair weights", (torch.float32,), True), self._stream()))
 
-    def experts_down(self, inner, chosen, weights, w_down, hidden):
-        """hidden[r] += sum_j weights[r, j] * Wd_e inner[r * top + j], e = chosen[r, j], j in order; w_down [E, D, ff]."""
+    def experts_down(self, inner, chosen, weights, w_down, hidden, fresh=False, through=None):
+        """hidden[r] += sum_j weights[r, j] * Wd_e inner[r * top + j], e = chosen[r, j], j in order; w_down [E, D, ff].  With
+        `through` [n, D] (of inner's type) the share of an expert numbered E or higher is through[r].  `fresh`: written, not added."""
         n_rows, top = chosen.shape
         experts, width, ff = w_down.shape
         if tuple(inner.shape) != (n_rows * top, ff) or tuple(hidden.shape) != (n_rows, width) or (weights is not None and weights.shape != (n_rows, top)) \
-                or w_down.dtype != inner.dtype:
+                or w_down.dtype != inner.dtype or not self._goes_through(through, n_rows, width, inner.dtype):
             raise KernelError(f"experts_down: shapes inner {tuple(inner.shape)}, weights {tuple(w_down.shape)}, hidden {tuple(hidden.shape)} do not fit")
         self._check(self.lib.bh_experts_down(
             self._ptr(inner, "experts inner"), _code(inner, "experts inner"), self._ptr(chosen, "chosen", (torch.int32,)),
             self._ptr(weights, "route weights", (torch.float32,), True), self._ptr(w_down, "expert down"),
-            self._ptr(hidden, "experts hidden", (torch.float32,)), n_rows, top, ff, width, self._stream()))
+            self._ptr(hidden, "experts hidden", (torch.float32,)), self._ptr(through, "experts input", None, True), n_rows, top, experts,
+            ff, width, int(bool(fresh)), self._stream()))
+
+    @staticmethod
+    def _goes_through(through, n_rows, width, dtype=None):
+        return through is None or (isinstance(through, torch.Tensor) and tuple(through.shape) == (n_rows, width)
+                                   and (dtype is None or through.dtype == dtype))
 
     def experts_group(self, chosen, lists, counts):
         """lists[e, :counts[e]] = the pairs p = row * top + j with chosen[row, j] == e, in ascending order; chosen int32 [n, top],
@@ -1480,15 +1509,19 @@ class HipKernels(KernelSizes):
             self._ptr(place, "place", (torch.int32,)), experts, k, n_rows,
             self._ptr(in_weights, "pair weights", (torch.float32,), True), self._stream()))
 
-    def experts_combine(self, y, place, weights, hidden, top=None):
-        """hidden[r] += sum_j weights[r, j] * y[place[r * top + j]] (place None: y[r * top + j]), j in order; y f32 [pairs, D]."""
+    def experts_combine(self, y, place, weights, hidden, top=None, fresh=False, through=None, chosen=None, experts=0):
+        """hidden[r] += sum_j weights[r, j] * y[place[r * top + j]] (place None: y[r * top + j]), j in order; y f32 [pairs, D].
+        With `through` [n, D] the share of a pair with chosen[r, j] >= experts is through[r].  `fresh`: written, not added."""
         n_rows, top = weights.shape if weights is not None else (hidden.shape[0], int(top))      # no weights: every share counts once
-        if tuple(y.shape) != (n_rows * top, hidden.shape[1]) or hidden.shape[0] != n_rows or (place is not None and place.shape != (n_rows * top,)):
+        if tuple(y.shape) != (n_rows * top, hidden.shape[1]) or hidden.shape[0] != n_rows or (place is not None and place.shape != (n_rows * top,)) \
+                or not self._goes_through(through, n_rows, hidden.shape[1]) \
+                or (through is not None and (chosen is None or tuple(chosen.shape) != (n_rows, top) or experts < 1)):
             raise KernelError(f"experts_combine: shapes y {tuple(y.shape)}, hidden {tuple(hidden.shape)} do not fit")
         self._check(self.lib.bh_experts_combine(
             self._ptr(y, "experts y", (torch.float32,)), self._ptr(place, "place", (torch.int32,), True),
-            self._ptr(weights, "route weights", (torch.float32,), True), self._ptr(hidden, "experts hidden", (torch.float32,)), n_rows, top,
-            hidden.shape[1], self._stream()))
+            self._ptr(weights, "route weights", (torch.float32,), True), self._ptr(hidden, "experts hidden", (torch.float32,)),
+            self._ptr(through, "experts input", None, True), _code(through, "experts input") if through is not None else F32,
+            self._ptr(chosen, "chosen", (torch.int32,), True), int(experts), n_rows, top, hidden.shape[1], int(bool(fresh)), self._stream()))
 
     def clamped_glu(self, gate_up, out, limit, alpha, shift=1.0):
         """out = g' * sigmoid(alpha g') * (u' + shift) with g' = min(g, limit), u' = clamp(u, -limit, limit); gate_up [n, 2 ff] = [g | u]."""
@@ -1507,13 +1540,13 @@ class HipKernels(KernelSizes):
                                             int(bool(nontemporal)), self._ptr(sink, "sink"), ctypes.byref(count), self._stream()))
         return int(count.value)
 
-    def swiglu(self, gate_up, out):
-        """out[r, i] = silu(gate_up[r, i]) * gate_up[r, F + i]."""
+    def swiglu(self, gate_up, out, gate="silu"):
+        """out[r, i] = act(gate_up[r, i]) * gate_up[r, F + i], act as `gate` names it."""
         n_rows, width = out.shape
         if gate_up.shape != (n_rows, 2 * width) or gate_up.dtype != out.dtype:
             raise KernelError(f"swiglu: shapes {tuple(gate_up.shape)} -> {tuple(out.shape)} do not fit")
         self._check(self.lib.bh_swiglu(self._ptr(gate_up, "gate_up"), self._ptr(out, "swiglu out"),
-                                       _code(out, "swiglu out"), n_rows, width, self._stream()))
+                                       _code(out, "swiglu out"), n_rows, width, self.GATES[gate], self._stream()))
 
     def sample(self, logits, tokens, bad, temperature=None, top_k=None, top_p=None, uniform=None):
         """tokens[row] = argmax (temperature absent or <= 0) or a draw from the tempered, filtered

@@ -53,6 +53,33 @@ class ScaledEmbedding(Embedding):
         return hidden
 
 
+class NormedEmbedding(Embedding):
+    """hidden[t] = n / sqrt(mean(n^2) + eps) * w for n = E[token[t]]; the norm's result is the float32 residual, not rounded."""
+
+    def __init__(self, vocab: int, width: int, name: str, eps: float, norm_name: str):
+        super().__init__(vocab, width, name)
+        if not (eps > 0.0):
+            raise ValueError(f"RMSNorm epsilon must be positive, got {eps}")
+        self.eps, self.norm_name = float(eps), norm_name
+        self.norm_weight: torch.Tensor | None = None
+
+    def tensor_specs(self):
+        return super().tensor_specs() + [TensorSpec(self.norm_name, (self.width,), "norm")]
+
+    def load(self, get):
+        super().load(get)
+        self.norm_weight = get(self.norm_name)
+
+    def working_bytes(self, step) -> int:
+        return 2 * super().working_bytes(step)
+
+    def forward(self, ctx):
+        rows = super().forward(ctx)
+        hidden = ctx.new_f32(ctx.n_rows, self.width)
+        ctx.kernels.rmsnorm(rows, self.norm_weight, self.eps, hidden)
+        return hidden
+
+
 class LMHead:
     graph_safe = True      # forward reads only the step's device tensors
     graph_safe_rows = None # ... whatever the number of tokens a sequence brings

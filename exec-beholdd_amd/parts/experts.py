@@ -10,7 +10,10 @@ Variants, each a constructor parameter: `scoring="sigmoid"` weighs a chosen expe
 norming over the chosen); `weigh_input=True` puts the weight on the expert's input, out = sum expert(weight * h), which for
 these experts is a factor on the gate and up sums ahead of the activation (W (w h) = w (W h)); `limit`, `alpha` and `shift`
 shape the activation g' * sigmoid(alpha g') * (u' + shift), an infinite limit with alpha 1 and shift 0 being silu(g) * u; the
-shared expert is any feed-forward part.
+shared expert is any feed-forward part; `scoring="softmax_all"` weighs a chosen expert by its share of the softmax over all of
+them, not renormed over the chosen; `correction` adds a learned number to every expert's score for the choice alone, the
+weight is the score without it; `identity` more experts stand behind those with matrices, their output is the input h itself
+(no work, no tensors: `experts_combine` adds weight * h).
 
 The experts' matrices are kept stacked: gate and up rows of an expert in one [2 ff, width] block, [experts, ...] in
 all.  The (row, choice) pairs are grouped by expert on the device (`experts_group`).  A step of few rows then runs a
@@ -77,6 +80,7 @@ class ClampedGLU:
 class RoutedExperts:
     graph_safe = True
     graph_safe_rows = 1       # steps of several rows a sequence may read the experts' counts on the host
+    writes_fresh = True       # forward(..., fresh=True) writes its result instead of adding it
     PRODUCT_PAIRS = 16        # from that many pairs an expert on average, a step of many rows runs matrix products
     PACK_FOR_PROMPTS = True   # keep a second copy of every expert's matrices in the form the products of many rows read fastest
     ONE_LAUNCH_WORK = 1.5e11  # up to that many operations a layer, a prompt's experts run as one launch over all of them: the
@@ -85,17 +89,22 @@ class RoutedExperts:
 
     def __init__(self, hidden: int, n_experts: int, top: int, ff: int, limit: float, prefix: str, shared=None,
                  alpha: float = GATE_SLOPE, router_bias: bool = True, scoring: str = "softmax", weigh_input: bool = False,
-                 shift: float = 1.0):
-        if not 1 <= top <= n_experts:
-            raise ValueError(f"a row uses 1 to {n_experts} experts, got {top}")
-        if scoring not in ("softmax", "sigmoid"):
-            raise ValueError(f"experts are weighed by 'softmax' over the chosen or by each one's 'sigmoid', got {scoring!r}")
+                 shift: float = 1.0, identity: int = 0, correction: bool = False):
+        if not 1 <= top <= n_experts + identity:
+            raise ValueError(f"a row uses 1 to {n_experts + identity} experts, got {top}")
+        if scoring not in ("softmax", "sigmoid", "softmax_all"):
+            raise ValueError(f"experts are weighed by 'softmax' over the chosen, by each one's 'sigmoid' or by 'softmax_all', got {scoring!r}")
+        if correction and scoring != "softmax_all":
+            raise ValueError("a correction of the choice goes with scores over all experts")
+        if identity and weigh_input:
+            raise ValueError("identity experts are weighed on their output")
+        self.identity, self.has_correction = int(identity), bool(correction)
         self.scoring, self.weigh_input, self.shift = scoring, bool(weigh_input), float(shift)
         self.hidden, self.n_experts, self.top, self.ff = int(hidden), int(n_experts), int(top), int(ff)
         self.limit, self.alpha, self.prefix, self.shared = float(limit), float(alpha), prefix, shared
-        self.router = Linear(hidden, n_experts, prefix + "router")
+        self.router = Linear(hidden, n_experts + self.identity, prefix + "router")
         self.has_router_bias = bool(router_bias)
-        self.router_bias = self.w_gate_up = self.w_down = None
+        self.router_bias = self.correction = self.w_gate_up = self.w_down = None
         self.for_products = None      # per expert (gate and up, down) as the matrix products take them
         self.in_one_launch = False    # a prompt's products run as one launch over all experts (kernels.experts_products)
 
@@ -103,6 +112,8 @@ class RoutedExperts:
         specs = self.router.tensor_specs()
         if self.has_router_bias:
             specs.append(TensorSpec(self.prefix + "router.b", (self.n_experts,), "linear"))
+        if self.has_correction:
+            specs.append(TensorSpec(self.prefix + "correction", (self.n_experts + self.identity,), "linear"))
         for e in range(self.n_experts):
             specs += [TensorSpec(f"{self.prefix}e{e}.gate", (self.ff, self.hidden), "linear"),
                       TensorSpec(f"{self.prefix}e{e}.up", (self.ff, self.hidden), "linear"),
@@ -112,6 +123,7 @@ class RoutedExperts:
     def load(self, get):
         self.router.load(get)
         self.router_bias = get(self.prefix + "router.b").to(torch.float32).contiguous() if self.has_router_bias else None
+        self.correction = get(self.prefix + "correction").to(torch.float32).contiguous() if self.has_correction else None
         first = get(f"{self.prefix}e0.gate")
         self.w_gate_up = torch.empty((self.n_experts, 2 * self.ff, self.hidden), dtype=first.dtype, device=first.device)
         self.w_down = torch.empty((self.n_experts, self.hidden, self.ff), dtype=first.dtype, device=first.device)
@@ -142,24 +154,33 @@ class RoutedExperts:
             total += step.matrix(pairs, self.hidden) + step.matrix(pairs, 2 * self.ff) + step.matrix(pairs, 1, 4)
         return total + (self.shared.working_bytes(step) if self.shared is not None else 0)
 
-    def forward(self, ctx, x, hidden, then_norm=None):
+    def forward(self, ctx, x, hidden, then_norm=None, fresh=False):
         k = ctx.kernels
         n = x.shape[0]
         logits = self.router.forward(ctx, x, out_dtype=torch.float32)
         chosen = torch.empty((n, self.top), dtype=torch.int32, device=ctx.device)
         weights = ctx.new_f32(n, self.top)
-        k.route_top_k(logits, self.router_bias, chosen, weights, **({"scoring": self.scoring} if self.scoring != "softmax" else {}))
+        routing = {"scoring": self.scoring} if self.scoring != "softmax" else {}
+        if self.correction is not None:
+            routing["correction"] = self.correction
+        k.route_top_k(logits, self.router_bias, chosen, weights, **routing)
         ctx.extras["routing"] = (chosen, weights)
         # where the weight goes: on the expert's input (the kernels that make gate and up take it) or on its output
         act = {} if self.shift == 1.0 else {"shift": self.shift}
         ahead = dict(act, in_weights=weights) if self.weigh_input else act
         behind = None if self.weigh_input else weights
         pairs = n * self.top
+        # what the kernels that add a row's shares up need to know beside them: whether they write or add, and whose share is h
+        adding = {"fresh": True} if fresh else {}
+        if self.identity:
+            adding["through"], adding["chosen"], adding["experts"] = x, chosen, self.n_experts
         takes = getattr(k, "experts_rows_take", None)
         if takes is None or not (takes(self.hidden) and takes(self.ff)):
             inner = ctx.new_activations(pairs, self.ff)
             k.experts_gate_up(x, chosen, self.w_gate_up, inner, self.limit, self.alpha, **ahead)
-            k.experts_down(inner, chosen, behind, self.w_down, hidden)
+            if self.identity:
+                adding.pop("chosen"), adding.pop("experts")      # this kernel has both
+            k.experts_down(inner, chosen, behind, self.w_down, hidden, **adding)
         else:
             lists = torch.empty((self.n_experts, n), dtype=torch.int32, device=ctx.device)
             counts = torch.empty((self.n_experts,), dtype=torch.int32, device=ctx.device)
@@ -169,21 +190,20 @@ class RoutedExperts:
                 k.experts_rows(x, self.top, lists, counts, self.w_gate_up, inner, gated=True, limit=self.limit, alpha=self.alpha, **ahead)
                 y = ctx.new_f32(pairs, self.hidden)
                 k.experts_rows(inner, 1, lists, counts, self.w_down, y)
-                self._combine(k, y, None, behind, hidden)
+                self._combine(k, y, None, behind, hidden, adding)
             else:
-                self._as_products(ctx, x, lists, counts, weights, hidden)
+                self._as_products(ctx, x, lists, counts, weights, hidden, adding)
         if self.shared is not None:
             self.shared.forward(ctx, x, hidden)
         return None
 
-
-    def _combine(self, k, y, place, weights, hidden):
+    def _combine(self, k, y, place, weights, hidden, adding):
         if weights is not None:
-            k.experts_combine(y, place, weights, hidden)
+            k.experts_combine(y, place, weights, hidden, **adding)
         else:
-            k.experts_combine(y, place, None, hidden, top=self.top)
+            k.experts_combine(y, place, None, hidden, top=self.top, **adding)
 
-    def _as_products(self, ctx, x, lists, counts, weights, hidden):
+    def _as_products(self, ctx, x, lists, counts, weights, hidden, adding):
         """Every expert's pairs as one stretch of rows through the framework's matrix products."""
         k = ctx.kernels
         act = {} if self.shift == 1.0 else {"shift": self.shift}
@@ -203,10 +223,11 @@ class RoutedExperts:
             tiles = torch.tensor([(e, first + at, min(128, count - at)) for e, (first, count) in enumerate(zip(starts, held))
                                   for at in range(0, count, 128)], dtype=torch.int32, device=ctx.device)
             inner = ctx.new_activations(pairs, self.ff)
-            k.experts_products(gathered, self.w_gate_up, tiles, inner, gated=True, limit=self.limit, alpha=self.alpha, **act)
             y = ctx.new_f32(pairs, self.hidden)
-            k.experts_products(inner, self.w_down, tiles, y)
-            self._combine(k, y, place, behind, hidden)
+            if len(tiles):      # (every choice of the step may have fallen on identity experts)
+                k.experts_products(gathered, self.w_gate_up, tiles, inner, gated=True, limit=self.limit, alpha=self.alpha, **act)
+                k.experts_products(inner, self.w_down, tiles, y)
+            self._combine(k, y, place, behind, hidden, adding)
             return
         both = ctx.new_activations(pairs, 2 * self.ff)
         for e, (first, count) in enumerate(zip(starts, held)):
@@ -218,7 +239,7 @@ class RoutedExperts:
         for e, (first, count) in enumerate(zip(starts, held)):
             if count:
                 k.gemm(inner[first:first + count], matrices[e][1], y[first:first + count])
-        self._combine(k, y, place, behind, hidden)
+        self._combine(k, y, place, behind, hidden, adding)
 
 
 @FEED_FORWARDS.register("routed_experts")
@@ -240,3 +261,12 @@ def _build_routed_silu_experts(config, layer_index, prefix, shared):
     common = SwiGLU(config.hidden, sizes.shared_ff, prefix + "mlp.shared.", names=names) if sizes.shared_ff else None
     return RoutedExperts(config.hidden, sizes.experts, sizes.top, sizes.expert_ff, float("inf"), prefix + "mlp.", shared=common,
                          alpha=1.0, router_bias=False, scoring="sigmoid", weigh_input=True, shift=0.0)
+
+
+@FEED_FORWARDS.register("routed_identity_experts")
+def _build_routed_identity_experts(config, layer_index, prefix, shared):
+    """Experts of the form Wd (silu(Wg h) * (Wu h)) and experts that hand h through, chosen by corrected softmax scores over all
+    of them and weighed by the scores as they are."""
+    sizes = config.layers[layer_index].mlp
+    return RoutedExperts(config.hidden, sizes.experts, sizes.top, sizes.expert_ff, float("inf"), prefix + "mlp.", alpha=1.0,
+                         router_bias=False, scoring="softmax_all", shift=0.0, identity=sizes.identity, correction=True)

@@ -8,8 +8,15 @@ keys seen within a chunk or a window, and a gate on the heads' outputs.
     softmax of q.k * scale; query head h reads key/value head h // (heads / kv_heads)
     out = Wo (heads * sigmoid(Wg x))
 
+Variants, each a constructor parameter: `values_are_keys` (no Wv: a value is the head's own key as projected, before norm and
+rotation; then vdim = dim); `head_norm_weights=False` (queries and keys over their root mean square, no weight; a turn keeps a
+head's length, so such a norm ahead of the rotation and one behind it are one computation); `sink` (every softmax sum holds
+one more term exp(sink), the same for all heads, with neither key nor value); `gate="head"` (one gate a head, Wg x has
+`heads` numbers).
+
 The four projections are one stacked product [q | k | v | g]; the biases are added, the heads normed and turned, and
-keys and values written into the pages by one kernel (`head_norm_rope_write`).  Keys have `dim` dimensions a head and
+keys and values written into the pages by one kernel (`head_norm_rope_write`).  A gate a head is applied by the attention
+kernels themselves where their heads are the values' own size.  Keys have `dim` dimensions a head and
 values `vdim`; both are cached as heads of one padded size (zeros beyond), which the paged attention kernels take as it
 is.  Chunks are counted from a sequence's position 0, so what a row sees does not depend on how a prompt was cut; the
 cache keeps a chunk's (or a window's) span of positions and gives older pages back.  Norm statistics, angles and the
@@ -36,9 +43,11 @@ class GatedAttention:
 
     def __init__(self, hidden: int, n_heads: int, n_kv_heads: int, dim: int, vdim: int, scale: float, prefix: str, *,
                  bias: bool = True, head_norm_eps: float | None = None, turned: int = 0, base: float = 10000.0,
-                 chunk: int = 0, window: int = 0, gate: bool = True, rotation: RotaryFrequencies | None = None,
-                 neighbours: bool = False):
-        """`head_norm_eps` None: no query and key norms; `turned` 0: no rotation; `chunk` and `window` 0: every earlier key."""
+                 chunk: int = 0, window: int = 0, gate=True, rotation: RotaryFrequencies | None = None,
+                 neighbours: bool = False, values_are_keys: bool = False, head_norm_weights: bool = True,
+                 sink: float | None = None):
+        """`head_norm_eps` None: no query and key norms; `turned` 0: no rotation; `chunk` and `window` 0: every earlier key;
+        `gate` one a value (True), one a head ("head") or none (False); `sink` None: nothing beside the keys in a sum."""
         if n_heads % n_kv_heads:
             raise ValueError(f"{n_heads} query heads do not group evenly into {n_kv_heads} kv heads")
         if chunk and window:
@@ -47,19 +56,30 @@ class GatedAttention:
             turned = rotation.dims
         if turned % 2 or turned > dim:
             raise ValueError(f"the rotation turns pairs of a head's {dim} dimensions, got {turned}")
+        if gate not in (False, True, "head"):
+            raise ValueError(f"a gate is absent, one a value (True) or one a head ('head'), got {gate!r}")
+        if values_are_keys and (vdim != dim or bias):
+            raise ValueError(f"values that are their keys have the keys' size {dim} (got {vdim}) and no bias")
+        if rotation is not None and rotation.magnitude != 1.0 and head_norm_eps is not None and not head_norm_weights:
+            raise ValueError("a rotation that changes lengths does not go with heads of unit root mean square")
         self.hidden, self.n_heads, self.n_kv_heads, self.dim, self.vdim = int(hidden), int(n_heads), int(n_kv_heads), int(dim), int(vdim)
         self.scale, self.prefix, self.bias, self.head_norm_eps = float(scale), prefix, bool(bias), head_norm_eps
         self.turned, self.chunk, self.window = int(turned), int(chunk), int(window)
         self.q_width, self.k_width, self.v_width = self.n_heads * self.dim, self.n_kv_heads * self.dim, self.n_kv_heads * self.vdim
-        self.qkv_width = self.q_width + self.k_width + self.v_width
+        self.values_are_keys, self.head_norm_weights = bool(values_are_keys), bool(head_norm_weights) and head_norm_eps is not None
+        self.qkv_width = self.q_width + self.k_width + (0 if self.values_are_keys else self.v_width)
         self.gate_width = self.n_heads * self.vdim
+        self.gate_per_head = gate == "head"
+        self.sink = None if sink is None else float(sink)
         self.pad = padded_head(dim, vdim)
         self.gate, self.neighbours = bool(gate), bool(neighbours)
         self.rotation = rotation if rotation is not None else (RotaryFrequencies(self.turned, base) if self.turned else None)
-        self.proj = Linear(hidden, [self.q_width, self.k_width, self.v_width] + ([self.gate_width] if self.gate else []),
-                           [prefix + "q", prefix + "k", prefix + "v"] + ([prefix + "g"] if self.gate else []))
+        slices = [(self.q_width, "q"), (self.k_width, "k")] + ([] if self.values_are_keys else [(self.v_width, "v")])
+        if self.gate:
+            slices.append((self.n_heads if self.gate_per_head else self.gate_width, "g"))
+        self.proj = Linear(hidden, [width for width, _ in slices], [prefix + name for _, name in slices], whole=16 if self.gate_per_head else 1)
         self.out = Linear(self.gate_width, hidden, prefix + "o")
-        self.q_norm = self.k_norm = self.qkv_bias = None
+        self.q_norm = self.k_norm = self.qkv_bias = self.sinks = None
 
     @property
     def input_reader(self):
@@ -70,7 +90,7 @@ class GatedAttention:
         if self.bias:
             specs += [TensorSpec(self.prefix + "q.b", (self.q_width,), "linear"), TensorSpec(self.prefix + "k.b", (self.k_width,), "linear"),
                       TensorSpec(self.prefix + "v.b", (self.v_width,), "linear")]
-        if self.head_norm_eps is not None:
+        if self.head_norm_weights:
             specs += [TensorSpec(self.prefix + "q.norm", (self.dim,), "norm"), TensorSpec(self.prefix + "k.norm", (self.dim,), "norm")]
         return specs
 
@@ -79,7 +99,9 @@ class GatedAttention:
         self.out.load(get)
         if self.bias:
             self.qkv_bias = torch.cat([get(self.prefix + name).to(torch.float32) for name in ("q.b", "k.b", "v.b")]).contiguous()
-        if self.head_norm_eps is not None:
+        if self.sink is not None:
+            self.sinks = torch.full((self.n_heads,), self.sink, dtype=torch.float32, device=self.proj.weight.device)
+        if self.head_norm_weights:
             self.q_norm = get(self.prefix + "q.norm").to(torch.float32).contiguous()
             self.k_norm = get(self.prefix + "k.norm").to(torch.float32).contiguous()
 
@@ -107,18 +129,24 @@ class GatedAttention:
         freq = self.rotation.frequencies(ctx.device) if self.rotation is not None else None
         turning = dict(neighbours=self.neighbours, magnitude=self.rotation.magnitude) if self.rotation is not None and (
             self.neighbours or self.rotation.magnitude != 1.0) else {}
+        if self.head_norm_eps is not None and not self.head_norm_weights:
+            turning["unit_norm"] = True
+        if self.values_are_keys:
+            turning["values_are_keys"] = True
+        sinking = dict(sinks=self.sinks) if self.sinks is not None else {}
         k.head_norm_rope_write(proj, 0, self.qkv_bias, self.q_norm, self.k_norm, self.head_norm_eps or 0.0, freq, self.turned,
                                ctx.positions, ctx.row_seq, q, cache.k_pages, cache.v_pages, cache.page_table, self.n_heads,
                                self.n_kv_heads, self.dim, self.vdim, self.pad, cache.writes, **turning)
         plain = not self.gate and self.pad == self.vdim      # the attended heads are the output projection's input as they are
         attended = ctx.new_activations(n, self.n_heads * self.pad, reader=self.out.reader() if plain else None)
         k.attention(q, attended, cache.k_pages, cache.v_pages, cache.page_table, ctx.row_seq, ctx.positions, self.n_heads,
-                    self.n_kv_heads, self.pad, self.scale, self.window, layout=ctx, chunk=self.chunk)
+                    self.n_kv_heads, self.pad, self.scale, self.window, layout=ctx, chunk=self.chunk, **sinking)
         if plain:
             gated = attended
         else:
             gated = ctx.new_activations(n, self.gate_width, reader=self.out.reader())
-            k.gate_heads(attended, self.pad, proj if self.gate else None, self.qkv_width, gated, self.n_heads, self.vdim)
+            k.gate_heads(attended, self.pad, proj if self.gate else None, self.qkv_width, gated, self.n_heads, self.vdim,
+                         **(dict(per_head=True) if self.gate_per_head else {}))
         self.out.forward(ctx, gated, out=hidden, accumulate=not fresh)
         return None
 
@@ -129,3 +157,13 @@ def _build_gated_attention(config, layer_index, prefix, shared):
     return GatedAttention(config.hidden, sizes.heads, sizes.kv_heads, sizes.dim, sizes.vdim, sizes.scale, prefix + "mix.",
                           bias=getattr(sizes, "bias", True), head_norm_eps=config.rms_eps, turned=sizes.rot_dims,
                           base=sizes.rot_base, chunk=getattr(sizes, "chunk", 0), window=getattr(sizes, "window", 0))
+
+
+@MIXERS.register("keyed_value_attention")
+def _build_keyed_value_attention(config, layer_index, prefix, shared):
+    """Values that are their keys, heads of unit root mean square, a sink of score 0, one gate a head."""
+    sizes = config.layers[layer_index].mixer
+    rotation = RotaryFrequencies(sizes.rot_dims, sizes.rot_base, slowed=sizes.rot_slowed) if sizes.rot_dims else None
+    return GatedAttention(config.hidden, sizes.heads, sizes.kv_heads, sizes.dim, sizes.dim, sizes.scale, prefix + "mix.", bias=False,
+                          head_norm_eps=config.rms_eps, head_norm_weights=False, values_are_keys=True, chunk=sizes.chunk, gate="head",
+                          rotation=rotation, neighbours=True, sink=0.0)

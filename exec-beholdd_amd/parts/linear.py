@@ -17,14 +17,17 @@ from .base import ProductReader
 class Linear:
     graph_safe = True      # forward reads only the step's device tensors
     graph_safe_rows = None # ... whatever the number of tokens a sequence brings
-    def __init__(self, in_features: int, out_features, names):
-        """`names` and `out_features` are one name and size, or equal-length lists to stack."""
+    def __init__(self, in_features: int, out_features, names, whole: int = 1):
+        """`names` and `out_features` are one name and size, or equal-length lists to stack.  `whole`: the stacked matrix gets
+        rows of zeros behind its last tensor up to a multiple of that many (16 for the products that work in blocks of 16 weight
+        rows); `out_features` counts them, and the outputs they make are zeros that nobody needs to read."""
         self.in_features = int(in_features)
         self.names = [names] if isinstance(names, str) else list(names)
         self.splits = [int(out_features)] if isinstance(out_features, int) else [int(o) for o in out_features]
         if len(self.names) != len(self.splits):
             raise ValueError("one output size per stacked tensor")
-        self.out_features = sum(self.splits)
+        self.padding = -sum(self.splits) % int(whole)
+        self.out_features = sum(self.splits) + self.padding
         self.weight = None          # a tensor, or the kernel library's packed form of it
         self.shared = False
 
@@ -33,12 +36,14 @@ class Linear:
 
     def load(self, get):
         pieces = [get(name) for name in self.names]
-        if len(pieces) == 1:
+        if len(pieces) == 1 and not self.padding:
             self.weight = pieces[0]
         else:
             dtype = pieces[0].dtype
             if any(p.dtype != dtype for p in pieces):
                 pieces = [p.to(torch.float32) for p in pieces]   # mixed storage: keep the wider one
+            if self.padding:
+                pieces.append(torch.zeros((self.padding, self.in_features), dtype=pieces[0].dtype, device=pieces[0].device))
             self.weight = torch.cat(pieces, dim=0).contiguous()
 
     def use(self, weight: torch.Tensor):

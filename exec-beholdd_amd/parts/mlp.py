@@ -1,8 +1,8 @@
-"""Dense SwiGLU feed-forward: out = Wd (silu(Wg x) * (Wu x)), added to the residual.
+"""Dense feed-forwards.  SwiGLU: out = Wd (silu(Wg x) * (Wu x)), added to the residual.
 
 crates/beholdd-model/src/qwen3moe/forward.rs:1270-1298 with silu(x) = x / (1 + exp(-x)) and no
 clamp (crates/beholdd-kernel/src/vecops.rs:91-110, limit 0 at forward.rs:1288).  The gate and
-up matrices are stacked so that one product computes both.
+up matrices are stacked so that one product computes both.  `GeGLUTanh` is the same with the tanh form of GELU on the gate.
 """
 
 from __future__ import annotations
@@ -16,6 +16,9 @@ class SwiGLU:
     graph_safe_rows = None # ... whatever the number of tokens a sequence brings
     prepares_next_norm = True      # the down projection can carry the norm that follows
     takes_prepared_input = True    # x goes to the gate/up product untouched
+    writes_fresh = True            # forward(..., fresh=True) writes its result instead of adding it
+    GATE = "silu"                  # the activation on the gate, as the kernel library names it
+
     def __init__(self, hidden: int, intermediate: int, prefix: str, names=("gate_proj.weight", "up_proj.weight", "down_proj.weight")):
         """`names`: what the gate, up and down matrices are called behind `prefix`."""
         self.hidden, self.intermediate = hidden, intermediate
@@ -42,15 +45,29 @@ class SwiGLU:
         return (activated + self.gate_up.working_bytes(step, step.rows, accumulate=True, swiglu=True)
                 + self.down.working_bytes(step, step.rows, accumulate=True, then_norm=True))
 
-    def forward(self, ctx, x, hidden, then_norm=None):
+    def forward(self, ctx, x, hidden, then_norm=None, fresh=False):
         activated = ctx.new_activations(x.shape[0], self.intermediate, reader=self.down.reader())
-        ctx.kernels.gemm_swiglu(x, self.gate_up.weight, activated)     # both products and the gate in one pass
+        # both products and the gate in one pass
+        ctx.kernels.gemm_swiglu(x, self.gate_up.weight, activated, **({} if self.GATE == "silu" else {"gate": self.GATE}))
+        if fresh:
+            self.down.forward(ctx, activated, out=hidden)
+            return None
         return self.down.add_into(ctx, activated, hidden, then_norm)
 
 
 @FEED_FORWARDS.register("swiglu")
 def _build_swiglu(config, layer_index, prefix, shared):
     return SwiGLU(config.hidden, config.intermediate, prefix + "mlp.")
+
+
+class GeGLUTanh(SwiGLU):
+    """out = Wd (gelu(Wg x) * (Wu x)), gelu(z) = z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))."""
+    GATE = "gelu_tanh"
+
+
+@FEED_FORWARDS.register("geglu_tanh")
+def _build_geglu_tanh(config, layer_index, prefix, shared):
+    return GeGLUTanh(config.hidden, config.layers[layer_index].mlp.ff, prefix + "mlp.", names=("gate", "up", "down"))
 
 
 class SquaredReLU:

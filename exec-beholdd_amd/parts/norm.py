@@ -43,6 +43,17 @@ class RMSNorm:
         """This norm as the product that completes its input may prepare it."""
         return NormRequest(self.weight, self.eps, reader)
 
+    def add_forward(self, ctx, hidden, result, reader=None, rounded: bool = True):
+        """hidden <- hidden + norm(result), row by row and in place, all of it float32.  Returns what a sublayer that reads the
+        new residual takes as its input: the residual itself where the activations are float32, else a copy rounded to the
+        activation type, written by the same kernel (in the form `reader` reads fastest); None when `rounded` says that
+        nobody reads one."""
+        out = None
+        if rounded and ctx.act_dtype != torch.float32:
+            out = ctx.new_activations(hidden.shape[0], self.width, reader=reader)
+        ctx.kernels.add_rmsnorm(hidden, result, self.weight, self.eps, out)
+        return hidden if rounded and out is None else out
+
 
 class ZeroCentredRMSNorm(RMSNorm):
     """RMSNorm whose stored weight lies around zero: y = x / sqrt(mean(x^2) + eps) * (1 + w).  The sum 1 + w is made

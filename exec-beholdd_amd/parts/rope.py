@@ -58,9 +58,14 @@ class RotaryFrequencies:
     Models").  With d(t) = dims ln(original / (2 pi t)) / (2 ln base), the pair whose wave turns t times within
     `original` positions, lo = max(floor(d(fast)), 0), hi = min(ceil(d(slow)), dims - 1) and
     ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1):  freq_i <- freq_i / factor * ramp_i + freq_i (1 - ramp_i),
-    and every cosine and sine is multiplied by `magnitude` = 0.1 ln(factor) + 1 (1.0 without a stretch)."""
+    and every cosine and sine is multiplied by `magnitude` = 0.1 ln(factor) + 1 (1.0 without a stretch).
 
-    def __init__(self, dims: int, base: float, stretch=None):
+    `slowed` = (factor, low, high, original) slows pairs down by the length of their wave, 2 pi / freq_i positions
+    (the scheme of Llama 3.1): with t = original freq_i / (2 pi), how often the wave fits into `original` positions, freq_i
+    stays where t > high, becomes freq_i / factor where t < low, and in between, with m = (t - low) / (high - low),
+    (1 - m) freq_i / factor + m freq_i.  Cosine and sine keep their size."""
+
+    def __init__(self, dims: int, base: float, stretch=None, slowed=None):
         if dims <= 0 or dims % 2:
             raise ValueError(f"rotary width must be positive and even, got {dims}")
         if not (base > 0.0):
@@ -73,11 +78,24 @@ class RotaryFrequencies:
                 raise ValueError(f"a stretch needs a positive factor, length and turn counts and a base other than 1, got {stretch!r}")
             self.stretch = (factor, original, fast, slow)
             self.magnitude = 0.1 * math.log(factor) + 1.0
+        self.slowed = None
+        if slowed is not None:
+            if stretch is not None:
+                raise ValueError("a rotation is stretched or slowed by wavelength, not both")
+            factor, low, high, original = (float(value) for value in slowed)
+            if not (factor > 0.0 and original > 0.0 and 0.0 <= low <= high):
+                raise ValueError(f"slow pairs need a positive factor and length and 0 <= low <= high, got {slowed!r}")
+            self.slowed = (factor, low, high, original)
         self._frequencies = None
 
     def values(self) -> np.ndarray:
         """The frequencies in float64, one per pair."""
         plain = np.array([self.base ** (-2.0 * i / self.dims) for i in range(self.dims // 2)], dtype=np.float64)
+        if self.slowed is not None:
+            factor, low, high, original = self.slowed
+            fits = original * plain / (2.0 * math.pi)
+            share = np.clip((fits - low) / (high - low), 0.0, 1.0) if high > low else (fits >= low).astype(np.float64)
+            return (1.0 - share) * plain / factor + share * plain
         if self.stretch is None:
             return plain
         factor, original, fast, slow = self.stretch

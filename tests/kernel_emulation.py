@@ -339,22 +339,35 @@ class TorchKernels:
         if rounded is not None:
             rounded.copy_(result.to(rounded.dtype))
 
+    def add_rmsnorm(self, hidden, y, weight, eps, rounded=None):
+        self.calls.append("add_rmsnorm")
+        inv = 1.0 / torch.sqrt((y.double() ** 2).mean(-1, keepdim=True) + eps)
+        result = hidden.double() + y.double() * inv * weight.double()
+        hidden.copy_(result.float())
+        if rounded is not None:
+            rounded.copy_(result.to(rounded.dtype))
+
     def gelu_tanh(self, x, out=None):
         self.calls.append("gelu_tanh")
         z = x.double()
         (x if out is None else out).copy_((0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))).to(x.dtype))
 
     def head_norm_rope_write(self, proj, first, bias, q_weight, k_weight, eps, freq, turned, positions, row_seq, q_out, k_pages,
-                             v_pages, page_table, n_heads, n_kv_heads, dim, vdim, pad, write_kv, neighbours=False, magnitude=1.0):
+                             v_pages, page_table, n_heads, n_kv_heads, dim, vdim, pad, write_kv, neighbours=False, magnitude=1.0,
+                             unit_norm=False, values_are_keys=False):
         self.calls.append("head_norm_rope_write")
         n = proj.shape[0]
-        q_width, k_width, v_width = n_heads * dim, n_kv_heads * dim, n_kv_heads * vdim
+        q_width, k_width, v_width = n_heads * dim, n_kv_heads * dim, 0 if values_are_keys else n_kv_heads * vdim
         x = proj[:, first:first + q_width + k_width + v_width].float()
         if bias is not None:
             x = x + bias.float()
         q = x[:, :q_width].reshape(n, n_heads, dim)
         k = x[:, q_width:q_width + k_width].reshape(n, n_kv_heads, dim)
-        v = x[:, q_width + k_width:].reshape(n, n_kv_heads, vdim)
+        v = k if values_are_keys else x[:, q_width + k_width:].reshape(n, n_kv_heads, vdim)
+        if unit_norm:
+            assert q_weight is None
+            unit = lambda t: (t.double() / torch.sqrt((t.double() ** 2).mean(-1, keepdim=True) + eps)).float()
+            q, k = unit(q), unit(k)
         if q_weight is not None:
             rms = lambda t, w: (t.double() / torch.sqrt((t.double() ** 2).mean(-1, keepdim=True) + eps) * w.double()).float()
             q, k = rms(q, q_weight), rms(k, k_weight)
@@ -463,9 +476,16 @@ class TorchKernels:
         g, u = g.clamp(max=limit), u.clamp(min=-limit, max=limit)
         return g * torch.sigmoid(alpha * g) * (u + shift)
 
-    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax"):
+    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax", correction=None):
         self.calls.append("route_top_k")
         z = logits.double() + (bias.double() if bias is not None else 0.0)
+        if scoring == "softmax_all":
+            shares = torch.softmax(z, dim=-1)
+            order = torch.argsort(-(shares + (correction.double() if correction is not None else 0.0)), dim=-1, stable=True)[:, :chosen.shape[1]]
+            chosen.copy_(order.to(torch.int32))
+            weights.copy_(torch.gather(shares, 1, order).float())
+            return
+        assert correction is None
         order = torch.argsort(-z, dim=-1, stable=True)[:, :chosen.shape[1]]
         chosen.copy_(order.to(torch.int32))
         picked = torch.gather(z, 1, order)
@@ -476,19 +496,23 @@ class TorchKernels:
         top, ff = chosen.shape[1], w_gate_up.shape[1] // 2
         for row in range(h.shape[0]):
             for j in range(top):
+                if int(chosen[row, j]) >= w_gate_up.shape[0]:
+                    continue
                 both = w_gate_up[int(chosen[row, j])].double() @ h[row].double()
                 if in_weights is not None:
                     both = both * float(in_weights[row, j])
                 inner[row * top + j] = self._clamped_glu(both[:ff], both[ff:], limit, alpha, shift).to(inner.dtype)
 
-    def experts_down(self, inner, chosen, weights, w_down, hidden):
+    def experts_down(self, inner, chosen, weights, w_down, hidden, fresh=False, through=None):
         self.calls.append("experts_down")
         top = chosen.shape[1]
         for row in range(hidden.shape[0]):
             total = torch.zeros(hidden.shape[1], dtype=torch.float64)
             for j in range(top):
-                total += (float(weights[row, j]) if weights is not None else 1.0) * (w_down[int(chosen[row, j])].double() @ inner[row * top + j].double())
-            hidden[row] += total.float()
+                e = int(chosen[row, j])
+                share = through[row].double() if e >= w_down.shape[0] else w_down[e].double() @ inner[row * top + j].double()
+                total += (float(weights[row, j]) if weights is not None else 1.0) * share
+            hidden[row] = total.float() + (0.0 if fresh else hidden[row])
 
     def experts_group(self, chosen, lists, counts):
         self.calls.append("experts_group")
@@ -521,12 +545,18 @@ class TorchKernels:
                 gathered[int(offsets[e]) + i] = row if in_weights is None else (row.float() * in_weights.reshape(-1)[pair]).to(x.dtype)
                 place[pair] = int(offsets[e]) + i
 
-    def experts_combine(self, y, place, weights, hidden, top=None):
+    def experts_combine(self, y, place, weights, hidden, top=None, fresh=False, through=None, chosen=None, experts=0):
         self.calls.append("experts_combine")
         n, top = weights.shape if weights is not None else (hidden.shape[0], int(top))
         index = (place if place is not None else torch.arange(n * top)).long().reshape(n, top)
         share = weights.double()[:, :, None] if weights is not None else 1.0
-        hidden.add_((share * y.double()[index]).sum(1).float())
+        if through is not None:      # places of pairs that pass their input were never written
+            passes = (chosen >= experts)[:, :, None]
+            given = torch.where(passes, through.double()[:, None, :], y.double()[torch.where(passes[:, :, 0], torch.zeros_like(index), index)])
+        else:
+            given = y.double()[index]
+        total = (share * given).sum(1).float()
+        hidden.copy_(total if fresh else hidden + total)
 
     def clamped_glu(self, gate_up, out, limit, alpha, shift=1.0):
         self.calls.append("clamped_glu")
@@ -560,17 +590,20 @@ class TorchKernels:
         self.calls.append("weighted_sum")
         out.copy_((a * x.double() + b * y.double()).float())
 
-    def gemm_swiglu(self, a, w, out):
+    def gemm_swiglu(self, a, w, out, gate="silu"):
         self.calls.append("gemm_swiglu")
         both = torch.empty(a.shape[0], w.shape[0], dtype=a.dtype)
         self.gemm(a, w, both)
-        self.swiglu(both, out)
+        self.swiglu(both, out, gate)
 
-    def swiglu(self, gate_up, out):
+    def swiglu(self, gate_up, out, gate="silu"):
         self.calls.append("swiglu")
         width = out.shape[1]
         g, u = gate_up[:, :width].float(), gate_up[:, width:].float()
-        out.copy_((g / (1 + torch.exp(-g)) * u).to(out.dtype))
+        if gate == "gelu_tanh":
+            out.copy_((0.5 * g * (1.0 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g ** 3))) * u).to(out.dtype))
+        else:
+            out.copy_((g / (1 + torch.exp(-g)) * u).to(out.dtype))
 
     def sample(self, logits, tokens, bad, temperature=None, top_k=None, top_p=None, uniform=None):
         self.calls.append("sample")
