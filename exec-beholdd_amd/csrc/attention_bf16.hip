@@ -26,6 +26,7 @@
 // lo_j .. pos_j.  Rows of a page beyond the last written key are never multiplied in: their
 // probabilities are zero and their V values are zeroed before use.
 #include "attention_bf16.h"
+#include <type_traits>
 
 // A decode step can hand the kernel the fused projection rows themselves (struct FusedQkv) instead of
 // finished queries and a cache that already holds the new keys: every workgroup then norms and rotates
@@ -33,13 +34,21 @@
 // the new value as one more page of a single visible key, and writes both into the cache for the steps
 // to come.  The keys that come from the cache end one position earlier.  This takes the place of the
 // launch of the norm/rotation/cache-write kernel.
+//
+// The rows' heads come in one of two forms.  Whole heads turned in split halves by tables over positions (FUSED 1: HeadPrep);
+// or the first `turned` dimensions in neighbouring pairs by cosines and sines of the step's rows (FUSED 2: PairPrep), with the
+// norm's weights optional, in rows of any stride whose values may be the projected keys themselves.
 struct FusedQkv {
-  const uint16_t* qkv;      // [rows][(H + 2 KVH) * head_dim], one row per sequence; null: queries and cache are ready
+  const uint16_t* qkv;      // one row per sequence: H heads of q from column 0; null: queries and cache are ready
+  int row_stride;           // elements from one row to the next
+  int k_first, v_first;     // where a row's keys and its values begin (the same column: a value is its raw key)
+  int turned;               // FUSED 2: how many of a head's first dimensions turn
+  int unit_norm;            // FUSED 2: without weights the heads are still brought to unit root mean square
   const void* q_weight;     // per-head RMSNorm weights [head_dim], or null for no norm
   const void* k_weight;
   int weight_f32;           // their element type: float32, else bfloat16
   float eps;
-  const float* cos_table;   // [positions][head_dim / 2]: rotation over the whole head, or null for none
+  const float* cos_table;   // [positions][head_dim / 2]: rotation over the whole head (FUSED 2: [rows][turned / 2]), or null for none
   const float* sin_table;
   int write_kv;             // 0: the cache entry belongs to another layer, which has written the new key already
   uint16_t* k_pages;        // the cache again, to write into
@@ -81,6 +90,13 @@ struct HeadPrep {
     }
   }
 
+  __device__ inline void take_angles(const HeadPrep& other) {
+#pragma unroll
+    for (int s = 0; s < HS; ++s)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) cos_v[s][e] = other.cos_v[s][e], sin_v[s][e] = other.sin_v[s][e];
+  }
+
   // RMSNorm over the head, then split-half rotation: the partner of element i < HD / 2 is i + HD / 2, in the
   // same lane, HS slices on.
   __device__ inline void apply(float (&x)[NS][8], bool with_weight, int weight_f32, float eps, bool with_rotation) const {
@@ -115,6 +131,78 @@ struct HeadPrep {
   }
 };
 
+// The same for FUSED 2: a turned pair is dimensions 2i and 2i + 1, both in one lane; `row` is the row of the cosines and sines.
+template <int NS>
+struct PairPrep {
+  static constexpr int HD = 32 * NS;
+  u32x4_t weight_raw[NS][2];
+  float cos_v[NS][4], sin_v[NS][4];
+
+  __device__ inline void ask(const void* weight, int weight_f32) {
+    if (weight != nullptr) {
+#pragma unroll
+      for (int s = 0; s < NS; ++s) {
+        const int i = 32 * s + 8 * ((threadIdx.x % 64) / 16);
+        if (weight_f32) {
+          weight_raw[s][0] = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const float*>(weight) + i);
+          weight_raw[s][1] = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const float*>(weight) + i + 4);
+        } else {
+          weight_raw[s][0] = load16(reinterpret_cast<const uint16_t*>(weight) + i);
+        }
+      }
+    }
+  }
+  __device__ inline void ask_angles(const float* cos_rows, const float* sin_rows, int turned, int row, int g) {
+    const int half = turned / 2;
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+#pragma unroll
+      for (int p = 0; p < 4; ++p) {
+        const int pair = 16 * s + 4 * g + p;
+        cos_v[s][p] = pair < half ? cos_rows[(size_t)row * half + pair] : 1.f;
+        sin_v[s][p] = pair < half ? sin_rows[(size_t)row * half + pair] : 0.f;
+      }
+  }
+  __device__ inline void take_angles(const PairPrep& other) {
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+#pragma unroll
+      for (int p = 0; p < 4; ++p) cos_v[s][p] = other.cos_v[s][p], sin_v[s][p] = other.sin_v[s][p];
+  }
+  __device__ inline void apply(float (&x)[NS][8], bool with_norm, bool with_weight, int weight_f32, float eps, bool with_rotation) const {
+    if (with_norm) {
+      float ss = 0.f;
+#pragma unroll
+      for (int s = 0; s < NS; ++s)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += x[s][e] * x[s][e];
+      ss += __shfl_xor(ss, 16, 64);
+      ss += __shfl_xor(ss, 32, 64);
+      const float inv = 1.0f / sqrtf(ss / (float)HD + eps);
+#pragma unroll
+      for (int s = 0; s < NS; ++s)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          float w = 1.f;
+          if (with_weight)
+            w = weight_f32 ? __uint_as_float(weight_raw[s][e / 4][e % 4])
+                           : bf16_bits_to_f32((uint16_t)(weight_raw[s][0][e / 2] >> (16 * (e % 2))));
+          x[s][e] = x[s][e] * inv * w;
+        }
+    }
+    if (with_rotation) {
+#pragma unroll
+      for (int s = 0; s < NS; ++s)
+#pragma unroll
+        for (int p = 0; p < 4; ++p) {
+          const float a = x[s][2 * p], b = x[s][2 * p + 1];
+          x[s][2 * p] = a * cos_v[s][p] - b * sin_v[s][p];
+          x[s][2 * p + 1] = b * cos_v[s][p] + a * sin_v[s][p];
+        }
+    }
+  }
+};
+
 template <int NS>
 __device__ inline void widen_head(float (&x)[NS][8], const u32x4_t (&raw)[NS]) {
 #pragma unroll
@@ -133,18 +221,18 @@ __device__ inline void pack_head(u32x4_t (&out)[NS], const float (&x)[NS][8]) {
 
 // NS = head_dim / 32.
 // STREAM = one workgroup per (sequence, kv head, split): each cache byte is read once, past the caches.
-// FUSED = the step is a decode step and `fused.qkv` is given.
+// FUSED = the step is a decode step and `fused.qkv` is given, in form 1 or 2 (struct FusedQkv).
 // LEAN (with FUSED) = the queries are normed and rotated before the first page is asked for, and the new key's
 // numbers are asked for after the last page: nothing of that overlaps with the pages any more, but what it needs
 // in registers is gone while the pages stream, so that two workgroups fit a compute unit.  For launches of more
 // workgroups than compute units, where the second workgroup is worth more than the overlap.
-template <int NS, bool STREAM, bool FUSED, bool LEAN = false>
+template <int NS, bool STREAM, int FUSED, bool LEAN = false>
 __global__ __launch_bounds__(256, (LEAN ? 2 : 1)) void attention_mfma_kernel(
     const uint16_t* __restrict__ q, uint16_t* __restrict__ out, float* __restrict__ part_o,
     float* __restrict__ part_ml, const uint16_t* __restrict__ k_pages, const uint16_t* __restrict__ v_pages,
     const int32_t* __restrict__ page_table, int table_stride, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ seq_start, int H, int KVH, float scale_log2, int window, int n_splits,
-    int pages_per_split, int tile_groups, FusedQkv fused, int out_block_rows, const float* __restrict__ sinks) {
+    int pages_per_split, int tile_groups, FusedQkv fused, int out_block_rows, HeadEnd finish) {
   constexpr int HD = 32 * NS;
   __shared__ float sm_m[4][16];
   __shared__ float sm_l[4][16];
@@ -178,23 +266,33 @@ __global__ __launch_bounds__(256, (LEAN ? 2 : 1)) void attention_mfma_kernel(
   // loads are under way (q) and after the pages (the new key and value).
   u32x4_t q_raw[NS], k_raw[NS];
   uint16_t new_value[2 * NS];   // dim 16 dt + j of the new value
-  HeadPrep<NS> q_prep, k_prep;
+  std::conditional_t<FUSED == 2, PairPrep<NS>, HeadPrep<NS>> q_prep, k_prep;
   bool q_ready = !FUSED;
   const bool takes_new_key = FUSED && fused.write_kv && split == n_splits - 1 && wave == 0;
   auto ask_new_key = [&]() {   // one row per sequence: every lane's row is this row
-    const uint16_t* qkv_row = fused.qkv + (size_t)row * (H + 2 * KVH) * HD;
+    const uint16_t* qkv_row = fused.qkv + (size_t)row * fused.row_stride;
 #pragma unroll
-    for (int s = 0; s < NS; ++s) k_raw[s] = load16(qkv_row + (size_t)(H + kvh) * HD + 32 * s + 8 * g);
+    for (int s = 0; s < NS; ++s) k_raw[s] = load16(qkv_row + fused.k_first + kvh * HD + 32 * s + 8 * g);
 #pragma unroll
-    for (int dt = 0; dt < 2 * NS; ++dt) new_value[dt] = qkv_row[(size_t)(H + KVH + kvh) * HD + 16 * dt + j];
+    for (int dt = 0; dt < 2 * NS; ++dt) new_value[dt] = qkv_row[fused.v_first + kvh * HD + 16 * dt + j];
     // the rotation's numbers are q's, or (LEAN: q's are gone by then) asked for again
-    k_prep.ask(fused.k_weight, fused.weight_f32, LEAN ? fused.cos_table : nullptr, LEAN ? fused.sin_table : nullptr, pos_row, g);
+    if constexpr (FUSED == 2) {
+      k_prep.ask(fused.k_weight, fused.weight_f32);
+      if (LEAN && fused.cos_table) k_prep.ask_angles(fused.cos_table, fused.sin_table, fused.turned, row, g);
+    } else {
+      k_prep.ask(fused.k_weight, fused.weight_f32, LEAN ? fused.cos_table : nullptr, LEAN ? fused.sin_table : nullptr, pos_row, g);
+    }
   };
   if (FUSED) {
-    const uint16_t* qkv_row = fused.qkv + (size_t)row * (H + 2 * KVH) * HD;
+    const uint16_t* qkv_row = fused.qkv + (size_t)row * fused.row_stride;
 #pragma unroll
     for (int s = 0; s < NS; ++s) q_raw[s] = load16(qkv_row + (size_t)head * HD + 32 * s + 8 * g);
-    q_prep.ask(fused.q_weight, fused.weight_f32, fused.cos_table, fused.sin_table, pos_row, g);
+    if constexpr (FUSED == 2) {
+      q_prep.ask(fused.q_weight, fused.weight_f32);
+      if (fused.cos_table) q_prep.ask_angles(fused.cos_table, fused.sin_table, fused.turned, row, g);
+    } else {
+      q_prep.ask(fused.q_weight, fused.weight_f32, fused.cos_table, fused.sin_table, pos_row, g);
+    }
     if (takes_new_key && !LEAN) ask_new_key();
   } else {
     const uint16_t* qp = q + ((size_t)row * H + head) * HD + 8 * g;
@@ -204,7 +302,10 @@ __global__ __launch_bounds__(256, (LEAN ? 2 : 1)) void attention_mfma_kernel(
   auto finish_q = [&]() {
     float x[NS][8];
     widen_head<NS>(x, q_raw);
-    q_prep.apply(x, fused.q_weight != nullptr, fused.weight_f32, fused.eps, fused.cos_table != nullptr);
+    if constexpr (FUSED == 2)
+      q_prep.apply(x, fused.unit_norm || fused.q_weight != nullptr, fused.q_weight != nullptr, fused.weight_f32, fused.eps, fused.cos_table != nullptr);
+    else
+      q_prep.apply(x, fused.q_weight != nullptr, fused.weight_f32, fused.eps, fused.cos_table != nullptr);
     u32x4_t packed[NS];
     pack_head<NS>(packed, x);
 #pragma unroll
@@ -329,16 +430,11 @@ __global__ __launch_bounds__(256, (LEAN ? 2 : 1)) void attention_mfma_kernel(
     if (LEAN) ask_new_key();
     float x[NS][8];
     widen_head<NS>(x, k_raw);
-    if (!LEAN) {
-#pragma unroll
-      for (int s = 0; s < HeadPrep<NS>::HS; ++s)
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          k_prep.cos_v[s][e] = q_prep.cos_v[s][e];
-          k_prep.sin_v[s][e] = q_prep.sin_v[s][e];
-        }
-    }
-    k_prep.apply(x, fused.k_weight != nullptr, fused.weight_f32, fused.eps, fused.cos_table != nullptr);
+    if (!LEAN) k_prep.take_angles(q_prep);
+    if constexpr (FUSED == 2)
+      k_prep.apply(x, fused.unit_norm || fused.k_weight != nullptr, fused.k_weight != nullptr, fused.weight_f32, fused.eps, fused.cos_table != nullptr);
+    else
+      k_prep.apply(x, fused.k_weight != nullptr, fused.weight_f32, fused.eps, fused.cos_table != nullptr);
     u32x4_t new_key[NS];
     pack_head<NS>(new_key, x);
     const int token = pos_row % BH_PAGE;
@@ -402,8 +498,10 @@ __global__ __launch_bounds__(256, (LEAN ? 2 : 1)) void attention_mfma_kernel(
       const size_t column = (size_t)(row0 + cc / G) * H + kvh * G + cc % G;
       if (n_splits == 1) {   // out_block_rows: the output [rows][H * HD] lies in blocks of that many rows (bh_rows_index)
         // a sink: one more term exp(sinks[head]) in the softmax's sum (`top` is in powers of two)
-        if (sinks) sum += exp2f(sinks[kvh * G + cc % G] * 1.4426950408889634f - safe_top);
-        out[bh_rows_index(out_block_rows, row0 + cc / G, (kvh * G + cc % G) * HD + d, H * HD)] = f32_to_bf16_bits(value / sum);
+        const int out_row = row0 + cc / G, out_head = kvh * G + cc % G;
+        if (finish.sinks) sum += exp2f(finish.sinks[out_head] * 1.4426950408889634f - safe_top);
+        if (finish.gates) value *= head_gate<bf16_t>(finish, out_row, out_head);
+        out[bh_rows_index(out_block_rows, out_row, out_head * HD + d, H * HD)] = f32_to_bf16_bits(value / sum);
       } else {
         part_o[(column * n_splits + split) * HD + d] = value;
         if (d == 0) {
@@ -422,8 +520,9 @@ __global__ __launch_bounds__(256, (LEAN ? 2 : 1)) void attention_mfma_kernel(
 template <int WIDTH>
 __global__ void attention_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                          uint16_t* __restrict__ out, int n_splits, int HD, int H, int out_block_rows,
-                                         const float* __restrict__ sinks) {
+                                         HeadEnd finish) {
   const size_t column = blockIdx.x;
+  const float gate = head_gate<bf16_t>(finish, (int)(column / H), (int)(column % H));
   const float* ml = part_ml + column * n_splits * 2;
   const int lane = threadIdx.x % BH_WAVE;
   // the first splits' outputs are asked for beside the maxima and sums, not after them
@@ -439,8 +538,8 @@ __global__ void attention_combine_kernel(const float* __restrict__ part_o, const
   for (int s = lane; s < n_splits; s += BH_WAVE) sum += ml[2 * s + 1] * exp2f(ml[2 * s] - top);
 #pragma unroll
   for (int off = BH_WAVE / 2; off > 0; off >>= 1) sum += __shfl_xor(sum, off, BH_WAVE);
-  if (sinks) sum += exp2f(sinks[column % H] * 1.4426950408889634f - top);      // the sink's term, once for the whole row
-  const float inv = 1.0f / sum;
+  if (finish.sinks) sum += exp2f(finish.sinks[column % H] * 1.4426950408889634f - top);      // the sink's term, once for the whole row
+  const float inv = gate / sum;
   for (int d = threadIdx.x; d < HD; d += blockDim.x) {
     float value = 0.f;
     for (int s0 = 0; s0 < n_splits; s0 += WIDTH) {
@@ -513,8 +612,8 @@ static int attention_bf16_run(const void* q, void* out, void* part_o, void* part
                               const void* v_pages, const int32_t* page_table, int table_stride,
                               const int32_t* positions, const int32_t* seq_start, int n_seqs, int n_rows,
                               int max_rows_per_seq, int H, int KVH, int hd, float scale, int window,
-                              int max_position, int n_splits, const FusedQkv& fused, int out_blocked,
-                              const float* sinks, hipStream_t stream) {
+                              int max_position, int n_splits, const FusedQkv& fused, bool pairs, int out_blocked,
+                              const HeadEnd& finish, hipStream_t stream) {
   BH_REQUIRE(n_seqs > 0 && n_rows > 0 && max_rows_per_seq > 0, "attention_bf16: empty batch");
   BH_REQUIRE(H > 0 && KVH > 0 && H % KVH == 0, "attention_bf16: %d query heads do not group evenly into %d kv heads", H, KVH);
   BH_REQUIRE(hd % 32 == 0 && hd >= 32 && hd <= 256, "attention_bf16: head size %d is not a multiple of 32 up to 256", hd);
@@ -532,7 +631,7 @@ static int attention_bf16_run(const void* q, void* out, void* part_o, void* part
   if (!is_fused && n_splits == 1 && (long)tiles * KVH * n_seqs >= PREFILL_FROM_TILES) {   // many columns: the prefill kernel
     BH_REQUIRE(out_blocked == 0 || out_blocked == 16, "attention_bf16: a step of many columns writes rows or blocks of 16 rows, not of %d", out_blocked);
     bh_attention_prefill_launch(q, out, k_pages, v_pages, page_table, table_stride, positions, seq_start, n_seqs,
-                                tiles, H, KVH, hd, scale_log2, window, out_blocked == 16, sinks, stream);
+                                tiles, H, KVH, hd, scale_log2, window, out_blocked == 16, finish, stream);
     return bh_check_launch("attention_prefill_bf16");
   }
   BH_REQUIRE(out_blocked == 0 || ((out_blocked == 8 || out_blocked == 16) && (H * hd) % 32 == 0),
@@ -544,13 +643,15 @@ static int attention_bf16_run(const void* q, void* out, void* part_o, void* part
   attention_mfma_kernel<NS, STREAM, FUSED, ##__VA_ARGS__><<<grid, block, 0, stream>>>(                          \
       (const uint16_t*)q, (uint16_t*)out, (float*)part_o, (float*)part_ml, (const uint16_t*)k_pages,            \
       (const uint16_t*)v_pages, page_table, table_stride, positions, seq_start, H, KVH, scale_log2, window,     \
-      n_splits, per, tile_groups, fused, out_blocked, sinks)
+      n_splits, per, tile_groups, fused, out_blocked, finish)
 #define BH_ATT(NS)                                      \
   do {                                                  \
-    if (is_fused && lean && NS <= 4) BH_ATT_ONE(NS, true, true, (NS <= 4));   \
-    else if (is_fused) BH_ATT_ONE(NS, true, true);      \
-    else if (tile_groups == 1) BH_ATT_ONE(NS, true, false);  \
-    else BH_ATT_ONE(NS, false, false);                  \
+    if (pairs && lean && NS <= 4) BH_ATT_ONE(NS, true, 2, (NS <= 4));    \
+    else if (pairs) BH_ATT_ONE(NS, true, 2);            \
+    else if (is_fused && lean && NS <= 4) BH_ATT_ONE(NS, true, 1, (NS <= 4));   \
+    else if (is_fused) BH_ATT_ONE(NS, true, 1);         \
+    else if (tile_groups == 1) BH_ATT_ONE(NS, true, 0); \
+    else BH_ATT_ONE(NS, false, 0);                      \
   } while (0)
   switch (hd / 32) {
     case 1: BH_ATT(1); break;
@@ -569,10 +670,10 @@ static int attention_bf16_run(const void* q, void* out, void* part_o, void* part
     const dim3 columns(n_rows * H), threads(hd >= 128 ? 128 : 64);
     if (n_splits <= 4)
       attention_combine_kernel<4><<<columns, threads, 0, stream>>>((const float*)part_o, (const float*)part_ml, (uint16_t*)out,
-                                                                   n_splits, hd, H, out_blocked, sinks);
+                                                                   n_splits, hd, H, out_blocked, finish);
     else
       attention_combine_kernel<8><<<columns, threads, 0, stream>>>((const float*)part_o, (const float*)part_ml, (uint16_t*)out,
-                                                                   n_splits, hd, H, out_blocked, sinks);
+                                                                   n_splits, hd, H, out_blocked, finish);
     return bh_check_launch("attention_combine");
   }
   return 0;
@@ -582,11 +683,13 @@ extern "C" int bh_attention_bf16(const void* q, void* out, void* part_o, void* p
                                  const void* v_pages, const int32_t* page_table, int table_stride,
                                  const int32_t* positions, const int32_t* seq_start, int n_seqs, int n_rows,
                                  int max_rows_per_seq, int H, int KVH, int hd, float scale, int window,
-                                 int max_position, int n_splits, int out_blocked, const float* sinks, hipStream_t stream) {
-  const FusedQkv none = {nullptr, nullptr, nullptr, 0, 0.f, nullptr, nullptr, 0, nullptr, nullptr};
+                                 int max_position, int n_splits, int out_blocked, const float* sinks, const void* gates,
+                                 int gate_stride, hipStream_t stream) {
+  BH_REQUIRE(gates == nullptr || gate_stride >= H, "attention_bf16: a gate a head (%d) lies outside a row of %d", H, gate_stride);
+  const FusedQkv none = {};
   return attention_bf16_run(q, out, part_o, part_ml, k_pages, v_pages, page_table, table_stride, positions,
                             seq_start, n_seqs, n_rows, max_rows_per_seq, H, KVH, hd, scale, window, max_position,
-                            n_splits, none, out_blocked, sinks, stream);
+                            n_splits, none, false, out_blocked, HeadEnd{sinks, gates, gate_stride}, stream);
 }
 
 // A decode step (one row per sequence) straight from the fused projection rows [q heads | k heads | v heads]:
@@ -609,9 +712,55 @@ extern "C" int bh_attention_decode_fused(const void* qkv, void* out, void* part_
              "attention_decode_fused: the rotation must span the whole head (%d of %d) and the head be a multiple of 64", rot, hd);
   BH_REQUIRE(cos_table == nullptr || max_position < table_positions,
              "attention_decode_fused: position %d is outside the rotation table of %d positions", max_position, table_positions);
-  const FusedQkv fused = {(const uint16_t*)qkv, q_weight, k_weight, w_dtype == BH_F32, eps, cos_table, sin_table,
-                          write_kv, (uint16_t*)k_pages, (uint16_t*)v_pages};
+  const FusedQkv fused = {(const uint16_t*)qkv, (H + 2 * KVH) * hd, H * hd, (H + KVH) * hd, hd, 0, q_weight, k_weight,
+                          w_dtype == BH_F32, eps, cos_table, sin_table, write_kv, (uint16_t*)k_pages, (uint16_t*)v_pages};
   return attention_bf16_run(nullptr, out, part_o, part_ml, k_pages, v_pages, page_table, table_stride, positions,
-                            seq_start, n_seqs, n_seqs, 1, H, KVH, hd, scale, window, max_position, n_splits, fused,
-                            out_block_rows, nullptr, stream);
+                            seq_start, n_seqs, n_seqs, 1, H, KVH, hd, scale, window, max_position, n_splits, fused, false,
+                            out_block_rows, HeadEnd{}, stream);
+}
+
+// The same for rows whose heads turn in neighbouring pairs: from column `first` of rows of row_stride elements H heads of q, then
+// KVH of k and (unless values_are_keys) KVH of v; norm weights float32 [hd], both or neither, or (unit_norm) a norm without;
+// cos_rows and sin_rows [n_seqs][turned / 2] for the rows' positions; sinks and gates as in struct HeadEnd.
+extern "C" int bh_attention_decode_pairs(const void* rows, int row_stride, int first, void* out, void* part_o, void* part_ml,
+                                         void* k_pages, void* v_pages, const int32_t* page_table, int table_stride,
+                                         const int32_t* positions, const int32_t* seq_start, int n_seqs, int H, int KVH, int hd,
+                                         float scale, int window, int max_position, int n_splits, const float* q_weight,
+                                         const float* k_weight, int unit_norm, float eps, const float* cos_rows,
+                                         const float* sin_rows, int turned, int values_are_keys, int write_kv, int out_block_rows,
+                                         const float* sinks, const void* gates, int gate_stride, hipStream_t stream) {
+  BH_REQUIRE(rows != nullptr && H > 0 && KVH > 0 && hd > 0, "attention_decode_pairs: the projection rows are required");
+  const int k_first = H * hd, v_first = values_are_keys ? k_first : (H + KVH) * hd;
+  BH_REQUIRE(first >= 0 && first % 8 == 0 && row_stride % 8 == 0 && ((uintptr_t)rows) % 16 == 0 && first + v_first + KVH * hd <= row_stride,
+             "attention_decode_pairs: q, k and v from column %d lie outside a row of %d, or not on 16 bytes", first, row_stride);
+  BH_REQUIRE((q_weight == nullptr) == (k_weight == nullptr) && !(unit_norm && q_weight), "attention_decode_pairs: both norm weights, or neither");
+  BH_REQUIRE((cos_rows == nullptr) == (sin_rows == nullptr) && (cos_rows == nullptr || (turned > 0 && turned % 2 == 0 && turned <= hd)),
+             "attention_decode_pairs: %d turned dimensions of %d and their cosines and sines", turned, hd);
+  BH_REQUIRE(gates == nullptr || gate_stride >= H, "attention_decode_pairs: a gate a head (%d) lies outside a row of %d", H, gate_stride);
+  const FusedQkv fused = {(const uint16_t*)rows + first, row_stride, k_first, v_first, turned, unit_norm, q_weight, k_weight,
+                          1, eps, cos_rows, sin_rows, write_kv, (uint16_t*)k_pages, (uint16_t*)v_pages};
+  return attention_bf16_run(nullptr, out, part_o, part_ml, k_pages, v_pages, page_table, table_stride, positions, seq_start,
+                            n_seqs, n_seqs, 1, H, KVH, hd, scale, window, max_position, n_splits, fused, true, out_block_rows,
+                            HeadEnd{sinks, gates, gate_stride}, stream);
+}
+
+// cos_rows, sin_rows [n_rows][pairs]: cosine and sine (times `magnitude`) of the float32 angle position * freq[pair], once a step for
+// all the layers that turn by these frequencies.
+__global__ __launch_bounds__(256) void row_angles_kernel(const int32_t* __restrict__ positions, const float* __restrict__ freq,
+                                                         float magnitude, float* __restrict__ cos_rows, float* __restrict__ sin_rows,
+                                                         int n_rows, int pairs) {
+  const size_t n = (size_t)n_rows * pairs;
+  for (size_t e = (size_t)blockIdx.x * blockDim.x + threadIdx.x; e < n; e += (size_t)gridDim.x * blockDim.x) {
+    const float angle = (float)positions[e / pairs] * freq[e % pairs];
+    cos_rows[e] = cosf(angle) * magnitude;
+    sin_rows[e] = sinf(angle) * magnitude;
+  }
+}
+
+extern "C" int bh_row_angles(const int32_t* positions, const float* freq, float magnitude, float* cos_rows, float* sin_rows, int n_rows,
+                             int pairs, hipStream_t stream) {
+  BH_REQUIRE(n_rows > 0 && pairs > 0, "row_angles: sizes must be positive");
+  const size_t blocks = ((size_t)n_rows * pairs + 255) / 256;
+  row_angles_kernel<<<(int)(blocks < 4096 ? blocks : 4096), 256, 0, stream>>>(positions, freq, magnitude, cos_rows, sin_rows, n_rows, pairs);
+  return bh_check_launch("row_angles");
 }

@@ -37,6 +37,18 @@ __device__ inline float gate_mul(float gate, float up, GateForm form) {
   return gate / (1.0f + expf(-gate * fmaf(form.cube, gate * gate, form.slope))) * up;
 }
 
+// ---- what an attention kernel does where a (row, head)'s sum is finished ---------------------------
+struct HeadEnd {
+  const float* sinks;   // [heads] or null: exp(sinks[head]) is one more term of the head's softmax sums, without key and value
+  const void* gates;    // [rows][gate_stride] in the activations' type, or null: a finished head times sigmoid(gates[row][head])
+  int gate_stride;
+};
+template <typename T>
+__device__ inline float head_gate(const HeadEnd& end, int row, int head) {
+  if (end.gates == nullptr) return 1.0f;
+  return 1.0f / (1.0f + expf(-to_f32(reinterpret_cast<const T*>(end.gates)[(size_t)row * end.gate_stride + head])));
+}
+
 // ---- reductions -------------------------------------------------------------------------
 
 __device__ inline float wave_sum(float v) {

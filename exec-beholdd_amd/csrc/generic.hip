@@ -741,7 +741,7 @@ __global__ __launch_bounds__(THREADS) void attention_generic_kernel(
     const T* __restrict__ q, T* __restrict__ out, const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     const int32_t* __restrict__ page_table, int table_stride, const int32_t* __restrict__ row_seq,
     const int32_t* __restrict__ positions, int H, int KVH, int hd, float scale, int window, int kv_order,
-    const float* __restrict__ sinks) {
+    HeadEnd finish) {
   extern __shared__ float smem[];
   float* qs = smem;                    // [hd]
   float* probs = qs + hd;              // [THREADS]
@@ -800,8 +800,8 @@ __global__ __launch_bounds__(THREADS) void attention_generic_kernel(
     float total = 0.f;
     for (int g = 0; g < n_groups; ++g) total += partial[g * hd + tid];
     // a sink: one more term exp(sinks[head]) in the softmax's sum, with no key and no value
-    const float all = sinks ? run_sum + expf(sinks[head] - run_max) : run_sum;
-    out[((size_t)row * H + head) * hd + tid] = from_f32<T>(total / all);
+    const float all = finish.sinks ? run_sum + expf(finish.sinks[head] - run_max) : run_sum;
+    out[((size_t)row * H + head) * hd + tid] = from_f32<T>(total / all * head_gate<T>(finish, row, head));
   }
 }
 
@@ -809,7 +809,9 @@ extern "C" int bh_attention_generic(const void* q, void* out, int dtype, const v
                                     const void* v_pages, const int32_t* page_table, int table_stride,
                                     const int32_t* row_seq, const int32_t* positions, int n_rows, int H,
                                     int KVH, int hd, float scale, int window, int kv_order, const float* sinks,
-                                    hipStream_t stream) {
+                                    const void* gates, int gate_stride, hipStream_t stream) {
+  BH_REQUIRE(gates == nullptr || gate_stride >= H, "attention: a gate a head (%d) lies outside a row of %d", H, gate_stride);
+  const HeadEnd finish = {sinks, gates, gate_stride};
   BH_REQUIRE(n_rows > 0 && H > 0 && KVH > 0 && hd > 0, "attention: sizes must be positive");
   BH_REQUIRE(H % KVH == 0, "attention: %d query heads do not group evenly into %d kv heads", H, KVH);
   BH_REQUIRE(hd <= 1024, "attention: head size %d is above the limit of 1024", hd);
@@ -822,7 +824,7 @@ extern "C" int bh_attention_generic(const void* q, void* out, int dtype, const v
 #define BH_AG(T, THREADS)                                                                                             \
   attention_generic_kernel<T, THREADS><<<grid, block, smem, stream>>>((const T*)q, (T*)out, (const T*)k_pages, (const T*)v_pages, \
                                                                       page_table, table_stride, row_seq, positions, H, KVH, hd,  \
-                                                                      scale, window, kv_order, sinks)
+                                                                      scale, window, kv_order, finish)
 #define BH_AG_SIZES(T)                        \
   do {                                        \
     if (threads == AG_THREADS) BH_AG(T, AG_THREADS); \

@@ -143,7 +143,7 @@ class KernelSizes:
             "bh_qk_norm_rope_cache_takes_sums": [i, i, i],
             "bh_gemm_bf16_bare_parts": [i, i, i, i],
             "bh_gemm_bf16_bare": [p, p, p, i, i, i, i, i, p],
-            "bh_attention_generic": [p, p, i, p, p, p, i, p, p, i, i, i, i, f, i, i, p, p],
+            "bh_attention_generic": [p, p, i, p, p, p, i, p, p, i, i, i, i, f, i, i, p, p, i, p],
             "bh_swiglu": [p, p, i, i, i, i, p],
             "bh_sample": [p, p, p, p, p, p, p, p, i, i, p],
             "bh_sample_scratch": [i, i],
@@ -154,11 +154,13 @@ class KernelSizes:
             "bh_gemm_bf16_then_norm": [p, p, p, i, i, i, i, p, i, f, p, p, i, i, p],
             "bh_rows_blocked": [p, p, i, i, i, i, p],
             "bh_gemm_bf16_finishes_norm": [i, i, i, i],
-            "bh_attention_bf16": [p, p, p, p, p, p, p, i, p, p, i, i, i, i, i, i, f, i, i, i, i, p, p],
+            "bh_attention_bf16": [p, p, p, p, p, p, p, i, p, p, i, i, i, i, i, i, f, i, i, i, i, p, p, i, p],
             "bh_attention_bf16_splits": [i, i, i, i, i],
             "bh_attention_bf16_writes_blocked": [i, i, i, i, i],
             "bh_attention_decode_fused": [p, p, p, p, p, p, p, i, p, p, i, i, i, i, f, i, i, i, p, p, i, f, p, p, i, i,
                                           i, i, p],
+            "bh_attention_decode_pairs": [p, i, i, p, p, p, p, p, p, i, p, p, i, i, i, i, f, i, i, i, p, p, i, f, p, p, i, i, i, i, p, p, i, p],
+            "bh_row_angles": [p, p, f, p, p, i, i, p],
             "bh_kv_order": [i, i],
             "bh_stream_read": [p, ctypes.c_long, i, i, p, p, p],
             "bh_streams_open": [p, p, i, i, i, p],
@@ -249,9 +251,20 @@ class KernelSizes:
             total += _rounded(m * 2 * n * act_size)
         return total
 
+    PAGE = _build.source_page_size()
+
+    @staticmethod
+    def furthest(max_position, window=0, chunk=0) -> int:
+        """The largest position an attention call plans its walk over the keys for: the step's, or, where a row sees only the
+        positions of a window or a chunk, that of a sequence of as many pages as the stretch that a workgroup's rows (16 at most,
+        one after the other) see together can touch."""
+        span = int(window) or int(chunk)
+        return min(int(max_position), span + 15 + KernelSizes.PAGE - 2) if span else int(max_position)
+
     def attention_working_bytes(self, n_rows, n_seqs, max_rows_per_seq, n_heads, n_kv_heads, head_dim, max_position,
-                                act_size) -> int:
+                                act_size, window=0, chunk=0) -> int:
         """Bytes that an attention call allocates: the partial results of its key splits."""
+        max_position = self.furthest(max_position, window, chunk)
         if act_size != 2 or head_dim % 32 or head_dim > 256:
             return 0
         n_splits = int(self.lib.bh_attention_bf16_splits(int(n_seqs), int(max_rows_per_seq), int(n_heads), int(n_kv_heads),
@@ -707,19 +720,22 @@ class HipKernels(KernelSizes):
             raise KernelError(f"{what}: the page table must be [sequences, pages]")
 
     def attention(self, q, out, k_pages, v_pages, page_table, row_seq, positions, n_heads, n_kv_heads, head_dim,
-                  scale, window=0, layout=None, chunk=0, sinks=None):
+                  scale, window=0, layout=None, chunk=0, sinks=None, gates=None, gate_first=0):
         """out[row, head] = softmax(q . K * scale) V over the keys of the row's sequence that the row
         may see: positions max(0, p - window + 1) .. p with a window, p - p % chunk .. p with chunks (counted from
         the sequence's position 0), else 0 .. p; not both.  `layout`, when given,
         says how rows group into sequences (seq_start int32 [n_seqs + 1] on the device, n_seqs,
         max_rows_per_seq, max_position), which the matrix-core kernel needs; rows of one sequence
         are consecutive and in position order.  `sinks` (float32 [n_heads]): exp(sinks[head]) is one more term of the
-        head's softmax sums, with no key and no value."""
+        head's softmax sums, with no key and no value.  `gates` [n, P] of q's type: a finished head is multiplied by
+        sigmoid(gates[row, gate_first + head])."""
         n_rows = q.shape[0]
+        gating = self._gates(gates, gate_first, n_rows, n_heads, q.dtype, "attention")
         if sinks is not None and (sinks.shape != (n_heads,) or sinks.dtype != torch.float32):
             raise KernelError(f"attention: one float32 sink a head ({n_heads}), got {tuple(sinks.shape)} of {sinks.dtype}")
         if window < 0 or chunk < 0 or (window and chunk):
             raise KernelError(f"attention: a window ({window}) or chunks ({chunk}) of a positive count of positions, not both")
+        furthest = self.furthest(layout.max_position, window, chunk) if layout is not None else 0
         if chunk:
             window = -int(chunk)      # the kernels' one number for both (csrc/layout.h: bh_first_visible)
         if q.shape != (n_rows, n_heads * head_dim) or tuple(out.shape) != tuple(q.shape) or out.dtype != q.dtype:
@@ -728,10 +744,10 @@ class HipKernels(KernelSizes):
         if isinstance(out, BlockedRows) and not (
                 q.dtype == torch.bfloat16 and layout is not None and head_dim % 32 == 0 and head_dim <= 256
                 and (out.block_rows == 16 or not self.lib.bh_attention_bf16_writes_blocked(
-                    int(layout.n_seqs), int(layout.max_rows_per_seq), n_heads, n_kv_heads, int(layout.max_position)))):
+                    int(layout.n_seqs), int(layout.max_rows_per_seq), n_heads, n_kv_heads, furthest))):
             rows_out = torch.empty(tuple(q.shape), dtype=q.dtype, device=self.device)   # this step's kernel writes rows
             self.attention(q, rows_out, k_pages, v_pages, page_table, row_seq, positions, n_heads, n_kv_heads, head_dim,
-                           scale, max(window, 0), layout, chunk, sinks)
+                           scale, max(window, 0), layout, chunk, sinks, gates, gate_first)
             self.to_blocked(rows_out, out)
             return
         if n_heads % n_kv_heads != 0:
@@ -747,8 +763,7 @@ class HipKernels(KernelSizes):
             if layout.seq_start.shape != (n_seqs + 1,) or page_table.shape[0] < n_seqs:
                 raise KernelError("attention: seq_start must have one entry per sequence and one more, and the page "
                                   "table a row per sequence")
-            n_splits = int(self.lib.bh_attention_bf16_splits(n_seqs, max_rows, n_heads, n_kv_heads,
-                                                                      int(layout.max_position)))
+            n_splits = int(self.lib.bh_attention_bf16_splits(n_seqs, max_rows, n_heads, n_kv_heads, furthest))
             part_o = part_ml = None
             if n_splits > 1:   # partial results of the key splits: scratch for this call only
                 part_o = torch.empty(n_rows * n_heads * n_splits * head_dim, dtype=torch.float32, device=self.device)
@@ -758,15 +773,83 @@ class HipKernels(KernelSizes):
                              self._ptr(v_pages, "v_pages"), self._ptr(page_table, "page_table", (torch.int32,)),
                              page_table.shape[1], self._ptr(positions, "positions", (torch.int32,)),
                              self._ptr(layout.seq_start, "seq_start", (torch.int32,)), n_seqs, n_rows, max_rows,
-                             n_heads, n_kv_heads, head_dim, float(scale), int(window), int(layout.max_position),
-                             n_splits, _block_rows(out), self._ptr(sinks, "sinks", (torch.float32,), True), self._stream()))
+                             n_heads, n_kv_heads, head_dim, float(scale), int(window), furthest,
+                             n_splits, _block_rows(out), self._ptr(sinks, "sinks", (torch.float32,), True), *gating, self._stream()))
             return
         self._check(self.lib.bh_attention_generic(
             *common, _code(q, "q"), self._ptr(k_pages, "k_pages"), self._ptr(v_pages, "v_pages"),
             self._ptr(page_table, "page_table", (torch.int32,)), page_table.shape[1],
             self._ptr(row_seq, "row_seq", (torch.int32,)), self._ptr(positions, "positions", (torch.int32,)),
             n_rows, n_heads, n_kv_heads, head_dim, float(scale), int(window), self.kv_order(k_pages.dtype, head_dim),
-            self._ptr(sinks, "sinks", (torch.float32,), True), self._stream()))
+            self._ptr(sinks, "sinks", (torch.float32,), True), *gating, self._stream()))
+
+    def _gates(self, gates, gate_first, n_rows, n_heads, dtype, what):
+        """(address of the first row's first gate, elements from row to row) of a matrix that holds a gate a head, or none."""
+        if gates is None:
+            return None, 0
+        if gates.dim() != 2 or gates.shape[0] != n_rows or gates.dtype != dtype or gate_first < 0 or gate_first + n_heads > gates.shape[1]:
+            raise KernelError(f"{what}: a gate a head from column {gate_first} of {tuple(gates.shape)} does not fit {n_rows} rows of {n_heads} heads")
+        return self._ptr(gates, f"{what} gates") + int(gate_first) * gates.element_size(), gates.shape[1]
+
+    def row_angles(self, positions, freq, magnitude, cos_rows, sin_rows):
+        """cos_rows, sin_rows f32 [n, pairs]: cosine and sine, times `magnitude`, of the float32 angle positions[r] * freq[pair]."""
+        n_rows, pairs = cos_rows.shape
+        if positions.shape != (n_rows,) or freq.shape != (pairs,) or sin_rows.shape != cos_rows.shape:
+            raise KernelError(f"row_angles: shapes positions {tuple(positions.shape)}, freq {tuple(freq.shape)}, out {tuple(cos_rows.shape)} do not fit")
+        f32 = (torch.float32,)
+        self._check(self.lib.bh_row_angles(self._ptr(positions, "positions", (torch.int32,)), self._ptr(freq, "frequencies", f32),
+                                           float(magnitude), self._ptr(cos_rows, "cosines", f32), self._ptr(sin_rows, "sines", f32),
+                                           n_rows, pairs, self._stream()))
+
+    def attention_decode_pairs_takes(self, dtype, head_dim, n_heads, n_kv_heads) -> bool:
+        """Whether `attention_decode_pairs` takes heads of these sizes (the rows of the step aside)."""
+        return (dtype == torch.bfloat16 and head_dim % 32 == 0 and head_dim <= 256 and n_heads % n_kv_heads == 0
+                and n_heads // n_kv_heads <= 16 and self.kv_order(dtype, head_dim) == 1)
+
+    def attention_decode_pairs(self, rows, first, out, q_weight, k_weight, eps, cos_rows, sin_rows, positions, k_pages, v_pages,
+                               page_table, n_heads, n_kv_heads, head_dim, scale, write_kv, layout, window=0, chunk=0,
+                               unit_norm=False, values_are_keys=False, sinks=None, gates=None, gate_first=0):
+        """`head_norm_rope_write` (neighbouring pairs, keys and values of one size) and `attention` in one launch for a step of one
+        row per sequence: rows [n, P] hold, from column `first`, the heads of q, k and (unless `values_are_keys`) v; cos_rows
+        and sin_rows f32 [n, turned / 2] (or None) are the rows' own.  `out` may be `BlockedRows`.  Returns False, having done
+        nothing, where the one kernel does not take the operands (then call the two)."""
+        n_rows = rows.shape[0]
+        if (layout is None or int(layout.max_rows_per_seq) != 1 or int(layout.n_seqs) != n_rows or rows.dtype != k_pages.dtype
+                or not self.attention_decode_pairs_takes(rows.dtype, head_dim, n_heads, n_kv_heads) or first % 8 or rows.shape[1] % 8):
+            return False
+        width = (n_heads + n_kv_heads * (1 if values_are_keys else 2)) * head_dim
+        if rows.dim() != 2 or first < 0 or first + width > rows.shape[1] or tuple(out.shape) != (n_rows, n_heads * head_dim) or out.dtype != rows.dtype:
+            raise KernelError(f"attention_decode_pairs: shapes rows {tuple(rows.shape)}, out {tuple(out.shape)} do not fit")
+        if positions.shape != (n_rows,) or layout.seq_start.shape != (n_rows + 1,) or page_table.shape[0] < n_rows:
+            raise KernelError("attention_decode_pairs: one position and one page-table row per sequence, and seq_start")
+        if (q_weight is None) != (k_weight is None) or any(w is not None and w.shape != (head_dim,) for w in (q_weight, k_weight)):
+            raise KernelError("attention_decode_pairs: one norm weight per dimension of a head, for queries and keys alike")
+        if (cos_rows is None) != (sin_rows is None) or (cos_rows is not None and (cos_rows.dim() != 2 or cos_rows.shape[0] != n_rows
+                                                                                  or cos_rows.shape != sin_rows.shape or 2 * cos_rows.shape[1] > head_dim)):
+            raise KernelError("attention_decode_pairs: a cosine and a sine per row and turned pair")
+        if sinks is not None and sinks.shape != (n_heads,):
+            raise KernelError(f"attention_decode_pairs: one sink a head ({n_heads}), got {tuple(sinks.shape)}")
+        if window < 0 or chunk < 0 or (window and chunk):
+            raise KernelError(f"attention_decode_pairs: a window ({window}) or chunks ({chunk}) of a positive count of positions, not both")
+        gating = self._gates(gates, gate_first, n_rows, n_heads, rows.dtype, "attention_decode_pairs")
+        self._check_pages(k_pages, v_pages, page_table, n_kv_heads, head_dim, rows.dtype, "attention_decode_pairs")
+        furthest = self.furthest(layout.max_position, window, chunk)
+        n_splits = int(self.lib.bh_attention_bf16_splits(n_rows, 1, n_heads, n_kv_heads, furthest))
+        part_o = part_ml = None
+        if n_splits > 1:
+            part_o = torch.empty(n_rows * n_heads * n_splits * head_dim, dtype=torch.float32, device=self.device)
+            part_ml = torch.empty(n_rows * n_heads * n_splits * 2, dtype=torch.float32, device=self.device)
+        f32, i32 = (torch.float32,), (torch.int32,)
+        self._check(self.lib.bh_attention_decode_pairs(
+            self._ptr(rows, "projection rows"), rows.shape[1], int(first), self._ptr(out, "attention out"),
+            self._ptr(part_o, "partial o", None, True), self._ptr(part_ml, "partial sums", None, True), self._ptr(k_pages, "k_pages"),
+            self._ptr(v_pages, "v_pages"), self._ptr(page_table, "page_table", i32), page_table.shape[1], self._ptr(positions, "positions", i32),
+            self._ptr(layout.seq_start, "seq_start", i32), n_rows, n_heads, n_kv_heads, head_dim, float(scale),
+            -int(chunk) if chunk else int(window), furthest, n_splits, self._ptr(q_weight, "q norm", f32, True),
+            self._ptr(k_weight, "k norm", f32, True), int(bool(unit_norm)), float(eps), self._ptr(cos_rows, "cosines", f32, True),
+            self._ptr(sin_rows, "sines", f32, True), 2 * cos_rows.shape[1] if cos_rows is not None else 0, int(bool(values_are_keys)),
+            int(bool(write_kv)), _block_rows(out), self._ptr(sinks, "sinks", f32, True), *gating, self._stream()))
+        return True
 
     def attention_decode_fused(self, qkv, out, q_weight, k_weight, eps, cos, sin, positions, k_pages, v_pages,
                                page_table, n_heads, n_kv_heads, head_dim, scale, window, write_kv, layout):

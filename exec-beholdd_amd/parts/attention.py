@@ -78,7 +78,7 @@ class GQAAttention:
         total += step.matrix(step.rows, q_width)                                                     # normed, rotated queries
         if step.sizes is not None:
             total += step.sizes.attention_working_bytes(step.rows, step.seqs, step.max_rows_per_seq, self.n_heads,
-                                                        self.n_kv_heads, self.head_dim, step.max_position, step.act_size)
+                                                        self.n_kv_heads, self.head_dim, step.max_position, step.act_size, window=self.window)
         return total + self.out.working_bytes(step, step.rows, accumulate=True, then_norm=True)
 
     def forward(self, ctx, x, hidden, cache, then_norm=None):

@@ -15,8 +15,10 @@ one more term exp(sink), the same for all heads, with neither key nor value); `g
 `heads` numbers).
 
 The four projections are one stacked product [q | k | v | g]; the biases are added, the heads normed and turned, and
-keys and values written into the pages by one kernel (`head_norm_rope_write`).  A gate a head is applied by the attention
-kernels themselves where their heads are the values' own size.  Keys have `dim` dimensions a head and
+keys and values written into the pages by one kernel (`head_norm_rope_write`); the attention kernels apply a gate a head
+themselves where their heads are the values' own size.  In a decode step, rows without biases whose heads turn in neighbouring
+pairs (or not at all) and need no padding go through one launch instead (`attention_decode_pairs`: norm, turn, cache write,
+attention, sink and gates), the cosines and sines of the step's rows made once for all layers that turn alike.  Keys have `dim` dimensions a head and
 values `vdim`; both are cached as heads of one padded size (zeros beyond), which the paged attention kernels take as it
 is.  Chunks are counted from a sequence's position 0, so what a row sees does not depend on how a prompt was cut; the
 cache keeps a chunk's (or a window's) span of positions and gives older pages back.  Norm statistics, angles and the
@@ -116,15 +118,33 @@ class GatedAttention:
     def working_bytes(self, step) -> int:
         total = self.proj.working_bytes(step, step.rows) + 2 * step.matrix(step.rows, self.n_heads * self.pad)
         total += step.matrix(step.rows, self.gate_width, reader=self.out.reader_for_plan(step.act_size))
+        if self.rotation is not None and step.rows <= step.seqs:      # a decode step's cosines and sines
+            total += 2 * step.matrix(step.rows, self.turned // 2, 4)
         if step.sizes is not None:
             total += step.sizes.attention_working_bytes(step.rows, step.seqs, step.max_rows_per_seq, self.n_heads, self.n_kv_heads,
-                                                        self.pad, step.max_position, step.act_size)
+                                                        self.pad, step.max_position, step.act_size, window=self.window, chunk=self.chunk)
         return total + self.out.working_bytes(step, step.rows, accumulate=True)
 
     def forward(self, ctx, x, hidden, cache, then_norm=None, fresh=False):
         k = ctx.kernels
         n = ctx.n_rows
         proj = self.proj.forward(ctx, x)
+        no_padding = self.pad == self.dim == self.vdim
+        # the attended heads are the output projection's input as they leave the attention kernel
+        plain = self.pad == self.vdim and (not self.gate or self.gate_per_head)
+        ending = dict(sinks=self.sinks) if self.sinks is not None else {}
+        if plain and self.gate_per_head:
+            ending.update(gates=proj, gate_first=self.qkv_width)
+        in_one = getattr(k, "attention_decode_pairs", None)
+        if (in_one is not None and ctx.is_decode and plain and no_padding and self.qkv_bias is None and (self.neighbours or self.rotation is None)
+                and k.attention_decode_pairs_takes(proj.dtype, self.pad, self.n_heads, self.n_kv_heads)):
+            cos, sin = self.rotation.row_angles(ctx) if self.rotation is not None else (None, None)
+            attended = ctx.new_activations(n, self.gate_width, reader=self.out.reader())
+            if in_one(proj, 0, attended, self.q_norm, self.k_norm, self.head_norm_eps or 0.0, cos, sin, ctx.positions, cache.k_pages, cache.v_pages,
+                      cache.page_table, self.n_heads, self.n_kv_heads, self.pad, self.scale, cache.writes, ctx, window=self.window, chunk=self.chunk,
+                      unit_norm=self.head_norm_eps is not None and not self.head_norm_weights, values_are_keys=self.values_are_keys, **ending):
+                self.out.forward(ctx, attended, out=hidden, accumulate=not fresh)
+                return None
         q = ctx.new_activations(n, self.n_heads * self.pad)
         freq = self.rotation.frequencies(ctx.device) if self.rotation is not None else None
         turning = dict(neighbours=self.neighbours, magnitude=self.rotation.magnitude) if self.rotation is not None and (
@@ -133,14 +153,12 @@ class GatedAttention:
             turning["unit_norm"] = True
         if self.values_are_keys:
             turning["values_are_keys"] = True
-        sinking = dict(sinks=self.sinks) if self.sinks is not None else {}
         k.head_norm_rope_write(proj, 0, self.qkv_bias, self.q_norm, self.k_norm, self.head_norm_eps or 0.0, freq, self.turned,
                                ctx.positions, ctx.row_seq, q, cache.k_pages, cache.v_pages, cache.page_table, self.n_heads,
                                self.n_kv_heads, self.dim, self.vdim, self.pad, cache.writes, **turning)
-        plain = not self.gate and self.pad == self.vdim      # the attended heads are the output projection's input as they are
         attended = ctx.new_activations(n, self.n_heads * self.pad, reader=self.out.reader() if plain else None)
         k.attention(q, attended, cache.k_pages, cache.v_pages, cache.page_table, ctx.row_seq, ctx.positions, self.n_heads,
-                    self.n_kv_heads, self.pad, self.scale, self.window, layout=ctx, chunk=self.chunk, **sinking)
+                    self.n_kv_heads, self.pad, self.scale, self.window, layout=ctx, chunk=self.chunk, **ending)
         if plain:
             gated = attended
         else:

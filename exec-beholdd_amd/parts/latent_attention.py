@@ -110,7 +110,7 @@ class LatentAttention:
             total += step.matrix(step.rows, self.query_rank) + self.query_up.working_bytes(step, step.rows)
         if step.sizes is not None:
             total += step.sizes.attention_working_bytes(step.rows, step.seqs, step.max_rows_per_seq, self.n_heads, 1,
-                                                        self.kv_head, step.max_position, step.act_size)
+                                                        self.kv_head, step.max_position, step.act_size, window=self.window)
         return total + self.out.working_bytes(step, step.rows, accumulate=True)
 
     def forward(self, ctx, x, hidden, cache, then_norm=None, fresh=False):

@@ -113,6 +113,16 @@ class RotaryFrequencies:
             self._frequencies = torch.from_numpy(self.values().astype(np.float32)).to(device).contiguous()
         return self._frequencies
 
+    def row_angles(self, ctx):
+        """(cosines, sines) float32 [rows, dims / 2] of the step's rows, times `magnitude`: made by the first layer of a step that
+        turns by these frequencies, found in `ctx.shared` by the others."""
+        key = ("row angles", self.dims, self.base, self.stretch, self.slowed)
+        if key not in ctx.shared:
+            cos, sin = ctx.new_f32(ctx.n_rows, self.dims // 2), ctx.new_f32(ctx.n_rows, self.dims // 2)
+            ctx.kernels.row_angles(ctx.positions, self.frequencies(ctx.device), self.magnitude, cos, sin)
+            ctx.shared[key] = (cos, sin)
+        return ctx.shared[key]
+
 
 class NoPositionEncoding:
     """For mixers whose order information comes from elsewhere (or nowhere)."""

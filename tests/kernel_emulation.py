@@ -75,7 +75,7 @@ class TorchKernels:
             v_pages[page, :, :, pos % PAGE] = v[row].to(v_pages.dtype)
 
     def attention(self, q, out, k_pages, v_pages, page_table, row_seq, positions, n_heads, n_kv_heads, head_dim,
-                  scale, window=0, layout=None, chunk=0, sinks=None):
+                  scale, window=0, layout=None, chunk=0, sinks=None, gates=None, gate_first=0):
         self.calls.append("attention")
         assert not (window and chunk)
         n_rows = q.shape[0]
@@ -97,6 +97,8 @@ class TorchKernels:
                 else:
                     probs = torch.softmax(scores, dim=0)
                 result[row, head] = (probs.double() @ values[:, kv, :].double()).float()
+        if gates is not None:
+            result = result * torch.sigmoid(gates[:, gate_first:gate_first + n_heads].float())[:, :, None]
         out.copy_(result.reshape(n_rows, n_heads * head_dim).to(out.dtype))
 
     def pack_weight(self, w):
