@@ -123,6 +123,7 @@ class DecoderModel:
         """Run one step.  `cache_for_run(i)` gives the LayerCache of the i-th scheduled run (or
         None); `want_rows` (int32 device tensor, may be empty) lists the rows whose logits are
         returned as float32 [len(want_rows), vocab]."""
+        ctx.shared.clear()      # a context that runs twice (launched, then captured) makes anew what its parts share
         hidden = self.embedding.forward(ctx)
         if self.residual is not None:
             hidden = self.residual.open(ctx, hidden)
@@ -136,6 +137,7 @@ class DecoderModel:
             if entering and run + 1 in self.pass_starts:
                 following = None      # the residual changes between the two blocks: nothing of the next norm can be made ahead
             prepared = self.blocks[layer].forward(ctx, hidden, cache_for_run(run), prepared, following)
+        ctx.shared.clear()
         if want_rows is None or want_rows.numel() == 0:
             return None
         reader = getattr(self.head, "input_reader", None) if getattr(self.final_norm, "serves_reader", False) else None

@@ -137,7 +137,7 @@ class StepContext:
     token_src: torch.Tensor | None = None  # int32 [T]: >= 0 where a row's token is fed_tokens[token_src[row]]
     fed_tokens: torch.Tensor | None = None # int32: tokens chosen on the device that the host has not read yet
     extras: dict = field(default_factory=dict)
-    shared: dict = field(default_factory=dict)   # what a part makes once a step for the parts after it (rotation angles of the rows)
+    shared: dict = field(default_factory=dict)   # what a part makes once a forward for the parts after it (rotation angles of the rows); emptied by the model at both ends
 
     def new_activations(self, *shape, reader=None):
         """An empty matrix of the activation type.  `reader` (a ProductReader) names the product that reads it
