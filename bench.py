@@ -76,8 +76,14 @@ def parse():
                              "Dupidra and Qwen3 at equal width and as many layer runs: prefill and decode tokens per second, and "
                              "every kernel of the new design beside its like with the fraction of its roofline; prints one JSON "
                              "line and exits")
+    parser.add_argument("--lurepel", action="store_true",
+                        help="the Lurepel design (attention within chunks whose values are its keys, heads of unit length, a sink and a "
+                             "gate a head; GELU-gated dense feed-forwards; experts chosen by corrected softmax scores, some of which "
+                             "hand their input through; norms on what the sublayers give) at layer sizes of real models beside "
+                             "Dupidra and Qwen3 at equal width and as many layers: prefill and decode tokens per second, and every "
+                             "kernel of the new design beside its like with the fraction of its roofline; prints one JSON line and exits")
     parser.add_argument("--alone", action="store_true",
-                        help="with --dupidra or --vepelix: the new design's two models only, without the models beside them and without the "
+                        help="with --dupidra, --vepelix or --lurepel: the new design's two models only, without the models beside them and without the "
                              "kernels timed alone (what a profiler should see of it)")
     parser.add_argument("--sampling", action="store_true",
                         help="time the selection kernel on 1, 8 and 64 rows of 151,936 logits (greedy, at a temperature, with "
@@ -1012,6 +1018,171 @@ def vepelix_bench(args, torch):
     return 0
 
 
+# ---- the Lurepel design beside Dupidra and Qwen3 at equal width and as many layers --------------------------------
+
+def lurepel_config(width, heads, vocab, experts=32, identity=8, top=4, chunk=4096):
+    """Eight layers: attention with heads of 128, four query heads to a key/value head, a rotation over half a head, six of them
+    within chunks of `chunk` positions and two over every earlier key; in turn a dense feed-forward three times the width and
+    `experts` experts of 3/8 of the width beside `identity` that hand their input through, of which `top` are used."""
+    def layer(index):
+        mixer = {"heads": heads, "kv_heads": max(heads // 4, 1), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                 "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+        if index % 4 != 3:
+            mixer["mask"] = {"size": chunk}
+        mlp = {"kind": "dense", "ff": 3 * width} if index % 2 == 0 else {
+            "kind": "moe", "router": {"experts": experts, "identity": identity, "top": top}, "expert": {"ff": 3 * width // 8}}
+        return {"type": "attention", "mixer": mixer, "mlp": mlp}
+
+    return {"architecture": "Lurepel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": [layer(index) for index in range(8)]}
+
+
+def lurepel_kernels(K, torch, width, heads, context):
+    """Every kernel that the design brought, and every older kernel in the turn the design gives it, beside its like among the
+    other models', alone, at a prompt of 2,048 rows and at a decode step of 8 rows over `context` cached tokens: microseconds and
+    the fraction of the roofline (the slower of its bytes at the HBM peak and its operations at the peak of the units it runs on)."""
+    from types import SimpleNamespace
+    bf16, dev = torch.bfloat16, "cuda:0"
+    dim, turned = 128, 64
+    page = K.page_size
+    out = {}
+
+    def note(name, us, n_bytes, flops=0.0, peak=PEAK_FLOPS["bf16"]):
+        floor = max(n_bytes / (PEAK_HBM_GBS * 1e9), flops / peak) * 1e6
+        out[name] = {"us": round(us, 1), "roofline_us": round(floor, 2), "fraction": round(floor / us, 3)}
+
+    kv_heads = max(heads // 4, 1)
+    q_w, k_w = heads * dim, kv_heads * dim
+    ones, head_weight, freq = torch.ones(width, device=dev), torch.ones(dim, device=dev), torch.ones(turned // 2, device=dev)
+    sinks, scale = torch.zeros(heads, device=dev), dim ** -0.5
+    for rows, seqs, past, tag in ((2048, 1, 0, "prompt of 2,048"), (8, 8, context - 1, f"decode of 8 at {context}")):
+        each = rows // seqs
+        starts = torch.arange(0, rows + 1, each, dtype=torch.int32, device=dev)
+        positions = (torch.arange(rows, dtype=torch.int32, device=dev) % each + past).contiguous()
+        row_seq = (torch.arange(rows, dtype=torch.int32, device=dev) // each).contiguous()
+        layout = SimpleNamespace(seq_start=starts, n_seqs=seqs, max_rows_per_seq=each, max_position=past + each - 1)
+        # -- the norm of what a sublayer gave, joined to the residual
+        hidden, result = torch.randn(rows, width, device=dev), torch.randn(rows, width, device=dev)
+        normed = torch.empty(rows, width, device=dev, dtype=bf16)
+        joined = 3 * hidden.numel() * 4 + normed.numel() * 2
+        us = timed(lambda: K.add_rmsnorm(hidden, result, ones, 1e-6, normed), torch)
+        note(f"add_rmsnorm, {tag}", us, joined)
+        us = timed(lambda: K.sum_layernorm(hidden, result, 2.0, ones, ones, 1e-6, normed), torch)
+        note(f"dupidra sum_layernorm, {tag}", us, joined)
+        # -- heads: unit norm, neighbour pairs, raw keys as values, cache write
+        proj = torch.randn(rows, q_w + k_w + heads, device=dev).to(bf16)
+        qkv = torch.randn(rows, q_w + 2 * k_w, device=dev).to(bf16)
+        per = -(-(past + each) // page)
+        k_pages = torch.randn(seqs * per, kv_heads, page, dim, device=dev).to(bf16)
+        v_pages = torch.randn(seqs * per, kv_heads, dim, page, device=dev).to(bf16)
+        table = torch.arange(seqs * per, dtype=torch.int32, device=dev).view(seqs, per).contiguous()
+        q_out = torch.empty(rows, q_w, device=dev, dtype=bf16)
+        us = timed(lambda: K.head_norm_rope_write(proj, 0, None, None, None, 1e-6, freq, turned, positions, row_seq, q_out, k_pages, v_pages, table,
+                                                  heads, kv_heads, dim, dim, dim, True, neighbours=True, unit_norm=True, values_are_keys=True), torch)
+        note(f"head_norm_rope_write, unit heads, neighbour pairs, keys as values, {tag}", us, rows * (2 * q_w + 3 * k_w) * 2)
+        us = timed(lambda: K.head_norm_rope_write(qkv, 0, None, head_weight, head_weight, 1e-6, freq, turned, positions, row_seq, q_out, k_pages,
+                                                  v_pages, table, heads, kv_heads, dim, dim, dim, True), torch)
+        note(f"dupidra head_norm_rope_write, {tag}", us, rows * (2 * q_w + 4 * k_w) * 2)
+        # -- attention with the sink and the gates in its ending, beside attention and gates in two launches
+        attended, gated = torch.empty_like(q_out), torch.empty_like(q_out)
+        for seen, what, kw in ((context, f"every key of a chunk of {context}", dict(chunk=-(-(past + each) // page) * page)), (4096, "chunks of 4,096", dict(chunk=4096))):
+            keys = seqs * min(past + each, seen) if each == 1 else each * (each + 1) // 2
+            n_bytes = 2 * seqs * min(past + each, seen) * k_w * 2 + 2 * q_out.numel() * 2
+            flops = 4.0 * keys * q_w
+            us = timed(lambda: K.attention(q_out, attended, k_pages, v_pages, table, row_seq, positions, heads, kv_heads, dim, scale, layout=layout,
+                                           sinks=sinks, gates=proj, gate_first=q_w + k_w, **kw), torch)
+            note(f"attention with sink and gates, {what}, {tag}", us, n_bytes, flops)
+            if each == 1:
+                cos, sin = (torch.ones(rows, turned // 2, device=dev) for _ in range(2))
+                us = timed(lambda: K.attention_decode_pairs(proj, 0, attended, None, None, 1e-6, cos, sin, positions, k_pages, v_pages, table, heads,
+                                                            kv_heads, dim, scale, True, layout, unit_norm=True, values_are_keys=True, sinks=sinks,
+                                                            gates=proj, gate_first=q_w + k_w, **kw), torch)
+                note(f"attention_decode_pairs (from the projection to gated heads), {what}, {tag}", us, n_bytes, flops)
+            us = timed(lambda: K.attention(q_out, attended, k_pages, v_pages, table, row_seq, positions, heads, kv_heads, dim, scale, layout=layout, **kw), torch)
+            note(f"dupidra attention, {what}, {tag}", us, n_bytes, flops)
+        wide_gate = torch.randn(rows, q_w, device=dev).to(bf16)
+        us = timed(lambda: K.gate_heads(attended, dim, wide_gate, 0, gated, heads, dim), torch)
+        note(f"dupidra gate_heads, {tag}", us, 3 * q_out.numel() * 2)
+        if each == 1:
+            cos_table = torch.ones(past + each, dim // 2, device=dev)
+            us = timed(lambda: K.attention_decode_fused(qkv, attended, head_weight, head_weight, 1e-6, cos_table, cos_table, positions, k_pages, v_pages,
+                                                        table, heads, kv_heads, dim, scale, 0, True, layout), torch)
+            note(f"qwen3 attention_decode_fused, {tag}", us, 2 * seqs * (past + each) * k_w * 2 + 2 * q_out.numel() * 2)
+            cos, sin = (torch.ones(rows, turned // 2, device=dev) for _ in range(2))
+            us = timed(lambda: K.row_angles(positions, freq, 1.0, cos, sin), torch)
+            note(f"row_angles (once a step), {tag}", us, 2 * cos.numel() * 4)
+        del k_pages, v_pages
+        # -- the dense feed-forward's first product with its gate
+        ff = 3 * width
+        weight = K.pack_weight(torch.randn(2 * ff, width, device=dev).to(bf16) * 0.02)
+        x = K.new_rows(rows, width, bf16, ff, True)
+        K.add_rmsnorm(hidden, result, ones, 1e-6, x)
+        activated = K.new_rows(rows, ff, bf16, width)
+        for name, gate in (("gelu gate", "gelu_tanh"), ("qwen3, silu gate", "silu")):
+            us = timed(lambda: K.gemm_swiglu(x, weight, activated, gate=gate), torch)
+            note(f"gate and up product, {name}, {tag}", us, 2 * ff * width * 2 + rows * (width + ff) * 2, 4.0 * rows * ff * width)
+        # -- routing and the experts
+        experts, identity, top, eff = 32, 8, 4, 3 * width // 8
+        logits = torch.randn(rows, experts + identity, device=dev)
+        correction = torch.randn(experts + identity, device=dev) * 0.01
+        chosen, shares = torch.empty(rows, top, dtype=torch.int32, device=dev), torch.empty(rows, top, device=dev)
+        plain_logits = logits[:, :experts].contiguous()
+        us = timed(lambda: K.route_top_k(plain_logits, None, chosen, shares), torch)
+        note(f"dupidra route_top_k, softmax over the chosen, {tag}", us, plain_logits.numel() * 4 + 2 * chosen.numel() * 4)
+        y = torch.randn(rows * top, width, device=dev)
+        us = timed(lambda: K.experts_combine(y, None, shares, hidden), torch)
+        note(f"dupidra experts_combine, {tag}", us, y.numel() * 4 + 2 * hidden.numel() * 4)
+        us = timed(lambda: K.route_top_k(logits, None, chosen, shares, scoring="softmax_all", correction=correction), torch)
+        note(f"route_top_k, corrected softmax over all, {tag}", us, logits.numel() * 4 + 2 * chosen.numel() * 4)
+        passing = float((chosen >= experts).float().mean())
+        rows_in = torch.randn(rows, width, device=dev).to(bf16)
+        us = timed(lambda: K.experts_combine(y, None, shares, hidden, fresh=True, through=rows_in, chosen=chosen, experts=experts), torch)
+        note(f"experts_combine with inputs handed through, {tag}", us, (1 - passing) * y.numel() * 4 + rows_in.numel() * 2 + hidden.numel() * 4)
+        if each == 1:
+            w_gu = torch.randn(experts, 2 * eff, width, device=dev).to(bf16) * 0.02
+            lists, counts = torch.empty(experts, rows, dtype=torch.int32, device=dev), torch.empty(experts, dtype=torch.int32, device=dev)
+            K.experts_group(chosen, lists, counts)
+            active = int((counts > 0).sum())
+            inner = torch.empty(rows * top, eff, device=dev, dtype=bf16)
+            for name, kw in (("silu", dict(limit=float("inf"), alpha=1.0, shift=0.0)), ("dupidra, clamped", dict(limit=7.0, alpha=1.702))):
+                us = timed(lambda: K.experts_rows(rows_in, top, lists, counts, w_gu, inner, gated=True, **kw), torch)
+                note(f"experts_rows gate and up, {name}, {tag}", us, active * 2 * eff * width * 2)
+    return out
+
+
+def lurepel_bench(args, torch):
+    from beholdd.engine import Engine, random_model_on_device
+
+    device, points = "cuda:0", []
+    t = min(args.prefill_tokens, args.context)
+    for width, heads in ((2048, 16), (4096, 32)):
+        models = {"lurepel": lurepel_config(width, heads, 32768), "dupidra": dupidra_config(width, heads, 32768),
+                  "qwen3": dict(QWEN3_8B, num_hidden_layers=8, hidden_size=width, num_attention_heads=heads,
+                                num_key_value_heads=heads // 4, intermediate_size=3 * width, vocab_size=32768)}
+        point = {"width": width, "heads": heads, "layer_runs": 8}
+        if args.alone:
+            models = {"lurepel": models["lurepel"]}
+        for name, config in models.items():
+            model = random_model_on_device(config, seed=0, dtype="bfloat16", device=device)
+            engine = Engine(model=model, dtype="bfloat16", max_tokens=args.batch * (-(-args.context // 64) * 64),
+                            max_slots=args.batch, device=device)
+            parameters = sum(int(np_prod(spec.shape)) for spec in model.tensor_specs())
+            seconds, _ = decode_run(engine, args.batch, args.context, args.steps, args.warmup, torch)
+            prefill = prefill_run(engine, t, torch)
+            point[name] = {"parameters": parameters, "decode_ms_per_step": round(seconds * 1e3, 4),
+                           "decode_tok_per_s": round(args.batch / seconds, 1), "prefill_ms": round(prefill * 1e3, 3),
+                           "prefill_tok_per_s": round(t / prefill, 1)}
+            kernels = engine.kernels
+            del engine, model
+            torch.cuda.empty_cache()
+        points.append(point)
+    line = {"metric": f"Lurepel beside Dupidra and Qwen3 at equal width and as many layers: decode tok/s @ batch {args.batch}, context {args.context}; prefill of {t} tokens",
+            "unit": "tok/s", "value": points[-1]["lurepel"]["decode_tok_per_s"], "dtype": "bf16", "data": "synthetic", "n_gpus": 1,
+            "steps": args.steps, "warmup": args.warmup, "higher_is_better": True, "points": points,
+            "kernels": {} if args.alone else lurepel_kernels(kernels, torch, 4096, 32, args.context)}
+    print(json.dumps(line))
+    return 0
+
+
 def np_prod(shape):
     total = 1
     for axis in shape:
@@ -1039,6 +1210,8 @@ def main():
         return dupidra_bench(args, torch)
     if args.vepelix:
         return vepelix_bench(args, torch)
+    if args.lurepel:
+        return lurepel_bench(args, torch)
 
     from beholdd.engine import Engine, random_model_on_device
 
