@@ -1117,6 +1117,7 @@ def lurepel_kernels(K, torch, width, heads, context):
         x = K.new_rows(rows, width, bf16, ff, True)
         K.add_rmsnorm(hidden, result, ones, 1e-6, x)
         activated = K.new_rows(rows, ff, bf16, width)
+        timed(lambda: K.gemm_swiglu(x, weight, activated), torch)      # (the clock settles under the matrix cores' load)
         for name, gate in (("gelu gate", "gelu_tanh"), ("qwen3, silu gate", "silu")):
             us = timed(lambda: K.gemm_swiglu(x, weight, activated, gate=gate), torch)
             note(f"gate and up product, {name}, {tag}", us, 2 * ff * width * 2 + rows * (width + ff) * 2, 4.0 * rows * ff * width)

@@ -22,36 +22,37 @@ __device__ inline float clamped_glu(float g, float u, float limit, float alpha, 
 }
 
 #define ROUTE_MAX_TOP 32
-#define ROUTE_PER_LANE 16      // experts a lane holds: up to 1024 experts
+#define ROUTE_PER_LANE 16      // experts a lane holds at most: up to 1024 experts
 
 // One wave a row: a lane holds the logits of experts lane, lane + 64, ...; the largest is found `top` times over, each time
-// without those already taken (ties go to the lower index).
-__global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restrict__ logits, const float* __restrict__ bias,
+// without those already taken (ties go to the lower index).  PER: experts a lane holds.
+template <int PER>
+__global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restrict__ logits, int stride, const float* __restrict__ bias,
                                                          const float* __restrict__ correction, int32_t* __restrict__ chosen,
                                                          float* __restrict__ weights, int n_rows, int E, int top, int scoring) {
   const int lane = threadIdx.x & (BH_WAVE - 1), row = blockIdx.x * (blockDim.x / BH_WAVE) + threadIdx.x / BH_WAVE;
   if (row >= n_rows) return;
-  const float* z = logits + (size_t)row * E;
-  float v[ROUTE_PER_LANE];
+  const float* z = logits + (size_t)row * stride;
+  float v[PER];
 #pragma unroll
-  for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+  for (int i = 0; i < PER; ++i) {
     const int e = lane + i * BH_WAVE;
     v[i] = e < E ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
   }
-  float score[ROUTE_PER_LANE];      // scoring 2: the share without the correction; v becomes the number to choose by
+  float score[PER];      // scoring 2: the share without the correction; v becomes the number to choose by
   if (scoring == 2) {
     float top_z = -INFINITY, total = 0.f;
 #pragma unroll
-    for (int i = 0; i < ROUTE_PER_LANE; ++i) top_z = fmaxf(top_z, v[i]);
+    for (int i = 0; i < PER; ++i) top_z = fmaxf(top_z, v[i]);
     top_z = wave_max(top_z);
 #pragma unroll
-    for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+    for (int i = 0; i < PER; ++i) {
       score[i] = lane + i * BH_WAVE < E ? expf(v[i] - top_z) : 0.f;
       total += score[i];
     }
     total = wave_sum(total);
 #pragma unroll
-    for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+    for (int i = 0; i < PER; ++i) {
       const int e = lane + i * BH_WAVE;
       score[i] /= total;
       if (e < E) v[i] = score[i] + (correction ? correction[e] : 0.f);
@@ -64,7 +65,7 @@ __global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restric
     float best = -INFINITY;
     int best_e = 0x7fffffff;
 #pragma unroll
-    for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+    for (int i = 0; i < PER; ++i) {
       const int e = lane + i * BH_WAVE;
       if (e < E && !((taken >> i) & 1u) && (v[i] > best || best_e == 0x7fffffff)) {
         best = v[i];
@@ -86,7 +87,7 @@ __global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restric
     if (scoring == 2) {
       float own = 0.f;
 #pragma unroll
-      for (int i = 0; i < ROUTE_PER_LANE; ++i)
+      for (int i = 0; i < PER; ++i)
         if (i == best_e / BH_WAVE) own = score[i];
       p = __shfl(own, best_e & (BH_WAVE - 1), BH_WAVE);
     } else {
@@ -104,12 +105,17 @@ __global__ __launch_bounds__(256) void route_top_k_kernel(const float* __restric
   }
 }
 
-extern "C" int bh_route_top_k(const float* logits, const float* bias, const float* correction, int32_t* chosen, float* weights, int n_rows, int E, int top,
+// logits [n_rows][stride]: a row's E logits are its first.
+extern "C" int bh_route_top_k(const float* logits, int stride, const float* bias, const float* correction, int32_t* chosen, float* weights, int n_rows, int E, int top,
                               int scoring, hipStream_t stream) {
   BH_REQUIRE(n_rows > 0 && E > 0 && E <= BH_WAVE * ROUTE_PER_LANE, "route_top_k: 1 to %d experts, got %d", BH_WAVE * ROUTE_PER_LANE, E);
+  BH_REQUIRE(stride >= E, "route_top_k: %d logits do not lie in a row of %d", E, stride);
   BH_REQUIRE(top >= 1 && top <= E && top <= ROUTE_MAX_TOP, "route_top_k: 1 to min(%d, %d) experts a row, got %d", E, ROUTE_MAX_TOP, top);
   BH_REQUIRE(scoring >= 0 && scoring <= 2 && (correction == nullptr || scoring == 2), "route_top_k: scoring %d, or a correction that does not go with it", scoring);
-  route_top_k_kernel<<<(n_rows + 3) / 4, 256, 0, stream>>>(logits, bias, correction, chosen, weights, n_rows, E, top, scoring);
+  const dim3 grid((n_rows + 3) / 4);
+  if (E <= BH_WAVE) route_top_k_kernel<1><<<grid, 256, 0, stream>>>(logits, stride, bias, correction, chosen, weights, n_rows, E, top, scoring);
+  else if (E <= 4 * BH_WAVE) route_top_k_kernel<4><<<grid, 256, 0, stream>>>(logits, stride, bias, correction, chosen, weights, n_rows, E, top, scoring);
+  else route_top_k_kernel<ROUTE_PER_LANE><<<grid, 256, 0, stream>>>(logits, stride, bias, correction, chosen, weights, n_rows, E, top, scoring);
   return bh_check_launch("route_top_k");
 }
 
@@ -411,6 +417,10 @@ __global__ __launch_bounds__(256) void experts_gather_kernel(const T* __restrict
     if (in_weights) {      // the pair's weight on the expert's input
       const float wgt = in_weights[pair];
       for (int k = threadIdx.x; k < K; k += blockDim.x) to[k] = from_f32<T>(to_f32(from[k]) * wgt);
+    } else if ((size_t)K * sizeof(T) % 16 == 0) {      // rows of whole 16-byte pieces
+      const uint4* pieces = reinterpret_cast<const uint4*>(from);
+      uint4* out = reinterpret_cast<uint4*>(to);
+      for (int k = threadIdx.x; k < (int)((size_t)K * sizeof(T) / 16); k += blockDim.x) out[k] = pieces[k];
     } else {
       for (int k = threadIdx.x; k < K; k += blockDim.x) to[k] = from[k];
     }
@@ -422,6 +432,7 @@ extern "C" int bh_experts_gather(const void* x, int dtype, int top, const int32_
                                  const int32_t* offsets, void* sorted, int32_t* place, int E, int K, int n_rows, const float* in_weights,
                                  hipStream_t stream) {
   BH_REQUIRE(E > 0 && K > 0 && top > 0 && n_rows > 0, "experts_gather: sizes must be positive");
+  BH_REQUIRE(((uintptr_t)x | (uintptr_t)sorted) % 16 == 0, "experts_gather: rows must be 16-byte aligned");
   dim3 grid(E, n_rows < 256 ? n_rows : 256);
   if (dtype == BH_F32)
     experts_gather_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, top, list, capacity, counts, offsets, (float*)sorted, place, K, in_weights);

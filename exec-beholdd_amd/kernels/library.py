@@ -194,7 +194,7 @@ class KernelSizes:
             "bh_gate_heads": [p, i, i, p, i, i, p, i, i, i, i, i, p],
             "bh_ssm_scan": [p, i, p, i, i, i, p, p, p, p, ctypes.c_long, p, p, p, i, i, i, i, i, p],
             "bh_gated_group_rmsnorm": [p, p, i, i, i, p, f, p, i, i, i, i, i, p],
-            "bh_route_top_k": [p, p, p, p, p, i, i, i, i, p],
+            "bh_route_top_k": [p, i, p, p, p, p, i, i, i, i, p],
             "bh_experts_gate_up": [p, i, p, p, p, i, i, i, i, i, f, f, f, p, p],
             "bh_experts_down": [p, i, p, p, p, p, p, i, i, i, i, i, i, p],
             "bh_clamped_glu": [p, i, p, i, i, f, f, i, f, p],
@@ -1479,20 +1479,22 @@ class HipKernels(KernelSizes):
     # ---- routed experts ----
     SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_all": 2}
 
-    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax", correction=None):
+    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax", correction=None, experts=None):
         """chosen[r] = the `top` largest of logits[r] + bias (largest first, ties to the lower index), weights[r] = softmax over
         those alone; logits f32 [n, E], chosen int32 [n, top], weights f32 [n, top].
         `scoring` "sigmoid": weights[r] = the sigmoid of every chosen logit, each for itself.  "softmax_all": weights[r] = the
-        chosen ones' shares of the softmax over all E, and the choice goes by share + `correction` (f32 [E])."""
+        chosen ones' shares of the softmax over all E, and the choice goes by share + `correction` (f32 [E]).
+        `experts`: how many of a row's first columns are logits (all of them where it is not said)."""
         if scoring not in self.SCORINGS or (correction is not None and scoring != "softmax_all"):
             raise KernelError(f"route_top_k: scoring is one of {sorted(self.SCORINGS)} (a correction goes with 'softmax_all'), got {scoring!r}")
-        n_rows, experts = logits.shape
+        n_rows, stride = logits.shape
+        experts = int(experts) if experts is not None else stride
         top = chosen.shape[1]
         if chosen.shape != (n_rows, top) or weights.shape != (n_rows, top) or any(
                 t is not None and t.shape != (experts,) for t in (bias, correction)):
             raise KernelError(f"route_top_k: shapes logits {tuple(logits.shape)}, chosen {tuple(chosen.shape)} do not fit")
         self._check(self.lib.bh_route_top_k(
-            self._ptr(logits, "router logits", (torch.float32,)), self._ptr(bias, "router bias", (torch.float32,), True),
+            self._ptr(logits, "router logits", (torch.float32,)), stride, self._ptr(bias, "router bias", (torch.float32,), True),
             self._ptr(correction, "router correction", (torch.float32,), True), self._ptr(chosen, "chosen", (torch.int32,)), self._ptr(weights, "route weights", (torch.float32,)), n_rows, experts, top,
             self.SCORINGS[scoring], self._stream()))
 

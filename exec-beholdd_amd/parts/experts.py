@@ -83,6 +83,8 @@ class RoutedExperts:
     writes_fresh = True       # forward(..., fresh=True) writes its result instead of adding it
     PRODUCT_PAIRS = 16        # from that many pairs an expert on average, a step of many rows runs matrix products
     PACK_FOR_PROMPTS = True   # keep a second copy of every expert's matrices in the form the products of many rows read fastest
+    WIDE_ROUTER = 128         # a router of fewer outputs is kept with that many for steps of more than WIDE_FROM_ROWS rows: products
+    WIDE_FROM_ROWS = 32       # that cut K into parts need a whole tile of outputs (2,048 rows, 40 experts: 71 -> 22 us)
     ONE_LAUNCH_WORK = 1.5e11  # up to that many operations a layer, a prompt's experts run as one launch over all of them: the
                               # one kernel reaches about 120 TFLOP/s whatever the size (tiles of 128 x 64 outputs re-read their
                               # operands through the L2), the products per expert cost about 25 us each and then run faster
@@ -103,6 +105,7 @@ class RoutedExperts:
         self.hidden, self.n_experts, self.top, self.ff = int(hidden), int(n_experts), int(top), int(ff)
         self.limit, self.alpha, self.prefix, self.shared = float(limit), float(alpha), prefix, shared
         self.router = Linear(hidden, n_experts + self.identity, prefix + "router")
+        self.router_wide = None       # the router's matrix with rows of zeros behind it, as the products of many rows take it
         self.has_router_bias = bool(router_bias)
         self.router_bias = self.correction = self.w_gate_up = self.w_down = None
         self.for_products = None      # per expert (gate and up, down) as the matrix products take them
@@ -138,6 +141,11 @@ class RoutedExperts:
         """The stacked matrices stay row after row (the kernels for steps of few rows read them so).  For prompts every expert's
         matrices are kept a second time in the kernel library's own form, where it has one for them: its products of many rows
         read that form several times as fast, and a GPU with hundreds of GB holds both."""
+        weight, widest = self.router.weight, self.WIDE_ROUTER
+        if hasattr(kernels, "packs") and kernels.packs(widest, self.hidden, weight.element_size()) and weight.shape[0] < widest:
+            wide = torch.zeros((widest, self.hidden), dtype=weight.dtype, device=weight.device)
+            wide[:weight.shape[0]].copy_(weight)
+            self.router_wide = kernels.pack_weight(wide)
         self.router.prepare(kernels)
         if self.shared is not None:
             self.shared.prepare(kernels)
@@ -147,7 +155,10 @@ class RoutedExperts:
             self.for_products = [(kernels.pack_weight(self.w_gate_up[e]), kernels.pack_weight(self.w_down[e])) for e in range(self.n_experts)]
 
     def working_bytes(self, step) -> int:
-        total = self.router.working_bytes(step, step.rows, out_size=4) + 2 * step.matrix(step.rows, self.top, 4)
+        total = self.router.working_bytes(step, step.rows, out_size=4)
+        if step.rows > self.WIDE_FROM_ROWS and self.router.out_features < self.WIDE_ROUTER:
+            total = step.matrix(step.rows, self.WIDE_ROUTER, 4) + step.product(step.rows, self.WIDE_ROUTER, self.hidden)
+        total += 2 * step.matrix(step.rows, self.top, 4)
         pairs = step.rows * self.top
         total += step.matrix(self.n_experts, step.rows, 4) + step.matrix(pairs, self.ff) + step.matrix(pairs, self.hidden, 4)
         if step.rows > step.seqs and pairs >= self.PRODUCT_PAIRS * self.n_experts:      # a step of many rows: the pairs' inputs, gate and up
@@ -157,10 +168,15 @@ class RoutedExperts:
     def forward(self, ctx, x, hidden, then_norm=None, fresh=False):
         k = ctx.kernels
         n = x.shape[0]
-        logits = self.router.forward(ctx, x, out_dtype=torch.float32)
+        routing = {"scoring": self.scoring} if self.scoring != "softmax" else {}
+        if self.router_wide is not None and n > self.WIDE_FROM_ROWS:
+            logits = ctx.new_f32(n, self.WIDE_ROUTER)
+            k.gemm(x, self.router_wide, logits)
+            routing["experts"] = self.router.out_features
+        else:
+            logits = self.router.forward(ctx, x, out_dtype=torch.float32)
         chosen = torch.empty((n, self.top), dtype=torch.int32, device=ctx.device)
         weights = ctx.new_f32(n, self.top)
-        routing = {"scoring": self.scoring} if self.scoring != "softmax" else {}
         if self.correction is not None:
             routing["correction"] = self.correction
         k.route_top_k(logits, self.router_bias, chosen, weights, **routing)

@@ -478,9 +478,9 @@ class TorchKernels:
         g, u = g.clamp(max=limit), u.clamp(min=-limit, max=limit)
         return g * torch.sigmoid(alpha * g) * (u + shift)
 
-    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax", correction=None):
+    def route_top_k(self, logits, bias, chosen, weights, scoring="softmax", correction=None, experts=None):
         self.calls.append("route_top_k")
-        z = logits.double() + (bias.double() if bias is not None else 0.0)
+        z = logits.double()[:, :experts] + (bias.double() if bias is not None else 0.0)
         if scoring == "softmax_all":
             shares = torch.softmax(z, dim=-1)
             order = torch.argsort(-(shares + (correction.double() if correction is not None else 0.0)), dim=-1, stable=True)[:, :chosen.shape[1]]
