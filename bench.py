@@ -1144,9 +1144,15 @@ def lurepel_kernels(K, torch, width, heads, context):
             K.experts_group(chosen, lists, counts)
             active = int((counts > 0).sum())
             inner = torch.empty(rows * top, eff, device=dev, dtype=bf16)
+            packed = K.pack_weight(w_gu.view(-1, width))
+            w_down = K.pack_weight(torch.randn(experts * width, eff, device=dev).to(bf16) * 0.02)
             for name, kw in (("silu", dict(limit=float("inf"), alpha=1.0, shift=0.0)), ("dupidra, clamped", dict(limit=7.0, alpha=1.702))):
-                us = timed(lambda: K.experts_rows(rows_in, top, lists, counts, w_gu, inner, gated=True, **kw), torch)
-                note(f"experts_rows gate and up, {name}, {tag}", us, active * 2 * eff * width * 2)
+                us = timed(lambda: K.experts_tiles(rows_in, top, lists, counts, packed, inner, gated=True, **kw), torch)
+                note(f"experts_tiles gate and up, {name}, {tag}", us, active * 2 * eff * width * 2)
+            us = timed(lambda: K.experts_rows(rows_in, top, lists, counts, w_gu, inner, gated=True, limit=7.0, alpha=1.702), torch)
+            note(f"experts_rows gate and up (the form for other sizes), {tag}", us, active * 2 * eff * width * 2)
+            us = timed(lambda: K.experts_tiles(inner, 1, lists, counts, w_down, y), torch)
+            note(f"experts_tiles down, {tag}", us, active * eff * width * 2)
     return out
 
 

@@ -206,6 +206,8 @@ class KernelSizes:
             "bh_experts_products_takes": [i, i],
             "bh_experts_group": [p, i, p, i, p, i, p],
             "bh_experts_rows": [p, i, i, p, i, p, p, p, i, i, i, i, f, f, f, p, p],
+            "bh_experts_tiles": [p, i, p, i, p, p, p, i, i, i, i, f, f, f, p, p],
+            "bh_experts_tiles_takes": [i, i],
             "bh_experts_gather": [p, i, i, p, i, p, p, p, p, i, i, i, p, p],
             "bh_gla_scan": [p, i, i, i, i, i, p, i, p, f, f, p, ctypes.c_long, p, p, p, i, i, i, i, i, i, i, p, p],
             "bh_gla_chunk_rows": [i, i, i, i, i],
@@ -1559,6 +1561,24 @@ class HipKernels(KernelSizes):
         self._check(self.lib.bh_experts_rows(
             self._ptr(rows, "experts rows"), _code(rows, "experts rows"), int(rows_per_pair_row), self._ptr(lists, "lists", (torch.int32,)),
             lists.shape[1], self._ptr(counts, "counts", (torch.int32,)), self._ptr(w, "expert weights"), self._ptr(out, "experts out"),
+            experts, k, n, int(bool(gated)), float(limit), float(alpha), float(shift),
+            self._ptr(in_weights, "pair weights", (torch.float32,), True), self._stream()))
+
+    def experts_tiles_take(self, dtype, inputs: int, outputs: int) -> bool:
+        """Whether `experts_tiles` takes products of these sizes and element type."""
+        return dtype == torch.bfloat16 and bool(self.lib.bh_experts_tiles_takes(int(inputs), int(outputs)))
+
+    def experts_tiles(self, rows, rows_per_pair_row, lists, counts, w, out, gated=False, limit=0.0, alpha=0.0, shift=1.0, in_weights=None):
+        """`experts_rows` on the matrix cores: `w` is the PackedWeight of all experts' matrices one below the other ([E * 2 N, K]
+        gated, gate rows and then up rows of every expert; otherwise [E * N, K])."""
+        experts, k = counts.shape[0], rows.shape[1]
+        n = out.shape[1]
+        if not isinstance(w, PackedWeight) or tuple(w.shape) != (experts * (2 if gated else 1) * n, k) or rows.dtype != torch.bfloat16 \
+                or out.dtype != (torch.bfloat16 if gated else torch.float32) or lists.shape[0] != experts:
+            raise KernelError(f"experts_tiles: shapes rows {tuple(rows.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)} do not fit")
+        self._check(self.lib.bh_experts_tiles(
+            self._ptr(rows, "experts rows", (torch.bfloat16,)), int(rows_per_pair_row), self._ptr(lists, "lists", (torch.int32,)), lists.shape[1],
+            self._ptr(counts, "counts", (torch.int32,)), self._ptr(w.data, "expert weights", (torch.bfloat16,)), self._ptr(out, "experts out"),
             experts, k, n, int(bool(gated)), float(limit), float(alpha), float(shift),
             self._ptr(in_weights, "pair weights", (torch.float32,), True), self._stream()))
 

@@ -17,8 +17,8 @@ weight is the score without it; `identity` more experts stand behind those with 
 
 The experts' matrices are kept stacked: gate and up rows of an expert in one [2 ff, width] block, [experts, ...] in
 all.  The (row, choice) pairs are grouped by expert on the device (`experts_group`).  A step of few rows then runs a
-workgroup per expert and block of outputs that reads the expert's rows from memory once for all of its pairs
-(`experts_rows`), with nothing that depends on the routing on the host, so that decode steps can be captured.  A step
+workgroup per expert and block of outputs that reads the expert's rows from memory once for all of its pairs (`experts_tiles`
+on the matrix cores from the packed form of the matrices, or `experts_rows` for sizes and element types that one does not take), with nothing that depends on the routing on the host, so that decode steps can be captured.  A step
 of many rows (a prompt) reads the experts' counts on the host (the step waits for the device there), lays the pairs'
 inputs side by side, expert after expert, and runs all experts' products in one launch on the matrix cores
 (`experts_products`, over a table of row tiles made from the counts; the activation rides in the first product), or,
@@ -109,6 +109,7 @@ class RoutedExperts:
         self.has_router_bias = bool(router_bias)
         self.router_bias = self.correction = self.w_gate_up = self.w_down = None
         self.for_products = None      # per expert (gate and up, down) as the matrix products take them
+        self.for_few_rows = None      # all experts' matrices one below the other, packed (gate and up, down), for kernels.experts_tiles
         self.in_one_launch = False    # a prompt's products run as one launch over all experts (kernels.experts_products)
 
     def tensor_specs(self):
@@ -151,7 +152,13 @@ class RoutedExperts:
             self.shared.prepare(kernels)
         takes = getattr(kernels, "experts_products_take", None)
         self.in_one_launch = bool(takes is not None and takes(self.w_gate_up.dtype, self.hidden, self.ff) and takes(self.w_down.dtype, self.ff, self.hidden))
-        if self.PACK_FOR_PROMPTS and hasattr(kernels, "pack_weight"):
+        tiles = getattr(kernels, "experts_tiles_take", None)
+        if tiles is not None and tiles(self.w_gate_up.dtype, self.hidden, self.ff) and tiles(self.w_down.dtype, self.ff, self.hidden):
+            self.for_few_rows = (kernels.pack_weight(self.w_gate_up.view(-1, self.hidden)), kernels.pack_weight(self.w_down.view(-1, self.ff)))
+            # blocks of 16 rows do not straddle experts: an expert's own packed matrices lie side by side in these
+            self.for_products = list(zip(*([type(whole)(part, whole.shape[0] // self.n_experts, whole.shape[1])
+                                            for part in whole.data.view(self.n_experts, -1)] for whole in self.for_few_rows)))
+        elif self.PACK_FOR_PROMPTS and hasattr(kernels, "pack_weight"):
             self.for_products = [(kernels.pack_weight(self.w_gate_up[e]), kernels.pack_weight(self.w_down[e])) for e in range(self.n_experts)]
 
     def working_bytes(self, step) -> int:
@@ -203,9 +210,10 @@ class RoutedExperts:
             k.experts_group(chosen, lists, counts)
             if ctx.is_decode or pairs < self.PRODUCT_PAIRS * self.n_experts:
                 inner = ctx.new_activations(pairs, self.ff)
-                k.experts_rows(x, self.top, lists, counts, self.w_gate_up, inner, gated=True, limit=self.limit, alpha=self.alpha, **ahead)
                 y = ctx.new_f32(pairs, self.hidden)
-                k.experts_rows(inner, 1, lists, counts, self.w_down, y)
+                product, (up, down) = (k.experts_tiles, self.for_few_rows) if self.for_few_rows is not None else (k.experts_rows, (self.w_gate_up, self.w_down))
+                product(x, self.top, lists, counts, up, inner, gated=True, limit=self.limit, alpha=self.alpha, **ahead)
+                product(inner, 1, lists, counts, down, y)
                 self._combine(k, y, None, behind, hidden, adding)
             else:
                 self._as_products(ctx, x, lists, counts, weights, hidden, adding)

@@ -340,6 +340,39 @@ def test_experts_some_of_which_hand_their_input_through(K, dtype, rows, width, e
         assert rel(got_shares.sort(dim=-1).values[sure], np.sort(shares[sure.numpy()], axis=-1)) < 1e-5
 
 
+@pytest.mark.parametrize("rows,experts,top,width,ff", [(1, 3, 1, 64, 16), (8, 32, 4, 2048, 768), (40, 2, 2, 256, 80), (33, 5, 3, 4096, 48), (5, 1, 1, 192, 1536)])
+@pytest.mark.parametrize("weighed", [False, True])
+def test_experts_of_few_rows_on_the_matrix_cores(K, rows, experts, top, width, ff, weighed):
+    """Both products of `experts_tiles` against the plain ones: experts without pairs, with more than sixteen (several passes over the
+    matrix), chunks that do not divide evenly over the waves; the gate's clamp and offset and a weight on the input."""
+    rng = np.random.default_rng(rows * experts)
+    x_t, x = rounded(rng.standard_normal((rows, width)), torch.bfloat16)
+    gu_t, gu = rounded(rng.standard_normal((experts, 2 * ff, width)) * 2 / np.sqrt(width), torch.bfloat16)
+    down_t, down = rounded(rng.standard_normal((experts, width, ff)) / np.sqrt(ff), torch.bfloat16)
+    chosen = np.stack([rng.permutation(experts)[:top] for _ in range(rows)]).astype(np.int32)
+    share = rng.uniform(0.2, 1.0, (rows, top)).astype(np.float32)
+    lists, counts = torch.empty(experts, rows, dtype=torch.int32, device="cuda:0"), torch.empty(experts, dtype=torch.int32, device="cuda:0")
+    K.experts_group(dev(chosen), lists, counts)
+    inner = torch.empty(rows * top, ff, dtype=torch.bfloat16, device="cuda:0")
+    K.experts_tiles(dev(x_t), top, lists, counts, K.pack_weight(dev(gu_t.reshape(-1, width))), inner, gated=True, limit=1.5, alpha=1.702, shift=1.0,
+                    in_weights=dev(share) if weighed else None)
+    want = np.zeros((rows * top, ff))
+    for r in range(rows):
+        for j in range(top):
+            both = gu[chosen[r, j]].astype(np.float64) @ x[r] * (share[r, j] if weighed else 1.0)
+            g, u = np.minimum(both[:ff], 1.5), np.clip(both[ff:], -1.5, 1.5)
+            want[r * top + j] = g * plain.sigmoid(1.702 * g) * (u + 1.0)
+    assert rel(inner, want) < 8e-3
+    y = torch.empty(rows * top, width, device="cuda:0")
+    if K.experts_tiles_take(torch.bfloat16, ff, width):
+        K.experts_tiles(inner, 1, lists, counts, K.pack_weight(dev(down_t.reshape(-1, ff))), y)
+    else:
+        K.experts_rows(inner, 1, lists, counts, dev(down_t), y)
+    held = inner.float().cpu().numpy()
+    for p in range(rows * top):
+        assert rel(y[p], down[chosen[p // top, p % top]].astype(np.float64) @ held[p]) < 2e-5, p
+
+
 def test_a_prompt_whose_choices_are_all_identity_experts(K, tmp_path):
     config = {"architecture": "Lurepel", "vocab": 50, "width": 128, "norm": {"eps": 1e-5},
               "layers": [lm.attention(2, 1, 32, 0.3, dims=8, mlp=lm.moe(2, 2, 64, identity=3)), lm.attention(2, 1, 32, 0.3, mlp=lm.dense(64))]}
