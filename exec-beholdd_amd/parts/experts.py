@@ -143,7 +143,8 @@ class RoutedExperts:
         matrices are kept a second time in the kernel library's own form, where it has one for them: its products of many rows
         read that form several times as fast, and a GPU with hundreds of GB holds both."""
         weight, widest = self.router.weight, self.WIDE_ROUTER
-        if hasattr(kernels, "packs") and kernels.packs(widest, self.hidden, weight.element_size()) and weight.shape[0] < widest:
+        if (isinstance(weight, torch.Tensor) and weight.shape[0] < widest and hasattr(kernels, "packs")
+                and kernels.packs(widest, self.hidden, weight.element_size())):
             wide = torch.zeros((widest, self.hidden), dtype=weight.dtype, device=weight.device)
             wide[:weight.shape[0]].copy_(weight)
             self.router_wide = kernels.pack_weight(wide)
@@ -221,13 +222,14 @@ class RoutedExperts:
             self.shared.forward(ctx, x, hidden)
         return None
 
-    def _combine(self, k, y, place, weights, hidden, adding):
+    def _combine(self, k, y, place, weights, hidden, adding=None):
+        adding = adding or {}
         if weights is not None:
             k.experts_combine(y, place, weights, hidden, **adding)
         else:
             k.experts_combine(y, place, None, hidden, top=self.top, **adding)
 
-    def _as_products(self, ctx, x, lists, counts, weights, hidden, adding):
+    def _as_products(self, ctx, x, lists, counts, weights, hidden, adding=None):
         """Every expert's pairs as one stretch of rows through the framework's matrix products."""
         k = ctx.kernels
         act = {} if self.shift == 1.0 else {"shift": self.shift}
