@@ -4,8 +4,8 @@ The reference's counterpart is its capture-and-compare tooling: `decode --logits
 (crates/beholdd-model/examples/decode.rs:78-82, :343-345) records logits and
 tools/compare_logits.py compares two captures.  This program instead takes the schedule from
 its input, so the same requests can be replayed whole, token by token, or in batches of
-unequal lengths, and every cut must give the same logits.  It has no forward pass, cache or
-loader of its own: it calls `Engine.step`.
+unequal lengths, and every cut must give the same logits.  All it does is call
+`Engine.step`: weights, cache and layers are the engine's.
 """
 
 from __future__ import annotations

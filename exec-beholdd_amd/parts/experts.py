@@ -12,8 +12,8 @@ these experts is a factor on the gate and up sums ahead of the activation (W (w 
 shape the activation g' * sigmoid(alpha g') * (u' + shift), an infinite limit with alpha 1 and shift 0 being silu(g) * u; the
 shared expert is any feed-forward part; `scoring="softmax_all"` weighs a chosen expert by its share of the softmax over all of
 them, not renormed over the chosen; `correction` adds a learned number to every expert's score for the choice alone, the
-weight is the score without it; `identity` more experts stand behind those with matrices, their output is the input h itself
-(no work, no tensors: `experts_combine` adds weight * h).
+weight is the score without it; `identity` more experts stand behind those with matrices and hand their input through
+(no tensors and no product: `experts_combine` adds weight * h).
 
 The experts' matrices are kept stacked: gate and up rows of an expert in one [2 ff, width] block, [experts, ...] in
 all.  The (row, choice) pairs are grouped by expert on the device (`experts_group`).  A step of few rows then runs a
